@@ -21,6 +21,7 @@ _SIGNATURES = {
     "imparo_pool_free": ([P, I], I), "imparo_pool_n_free": ([P], I), "imparo_pool_n_pages": ([P], I),
     "imparo_pool_high_water": ([P], I), "imparo_pool_is_free": ([P, I], I), "imparo_pool_scramble": ([P, c_uint64], I),
     "imparo_cache_new": ([I, P, I, P, I], P), "imparo_cache_delete": ([P], None),
+    "imparo_cache_keep_first": ([P, I, I], I),
     "imparo_cache_group_pool": ([P, I], P), "imparo_cache_slot_pool": ([P], P),
     "imparo_cache_admit": ([P, c_int64], I), "imparo_cache_release": ([P, c_int64], I),
     "imparo_cache_reserve": ([P, c_int64, I], I), "imparo_cache_rollback": ([P, c_int64], I),

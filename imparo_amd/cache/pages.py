@@ -13,7 +13,7 @@ twice is an error. The reference's block allocator keeps the same two rules
 from __future__ import annotations
 
 import ctypes
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from itertools import chain
 from typing import Dict, Hashable, Iterator, List, Optional, Sequence, Tuple, Union
 
@@ -114,7 +114,8 @@ class PagedSpec:
     as the mixer's kernels read them. `window` None keeps every position; a
     number keeps only that many. `chunk`: a query reads the positions of its
     own chunk only (chunks of that many positions, counted from position 0),
-    so the pages of earlier chunks are given back. Sites with equal specs share a pool and a
+    so the pages of earlier chunks are given back. `keep_first`: beside its
+    window a query reads the first so many positions, whose pages stay. Sites with equal specs share a pool and a
     block table per request. `fixed`: what the site keeps per request beside
     its pages, of a fixed size (the input its last token left, for a layer that
     mixes every token with the one before it)."""
@@ -122,8 +123,11 @@ class PagedSpec:
     window: Optional[int] = None
     fixed: Optional["FixedSpec"] = None
     chunk: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self):
+        if self.keep_first < 0 or (self.keep_first and self.window is None and self.chunk is None):
+            raise ValueError("the first positions are kept beside a window or a chunk, and their number is not negative")
         if self.chunk is not None and (self.window is not None or self.chunk < 1):
             raise ValueError("a paged spec keeps a window or the query's own chunk (of at least one position), not both")
         names = [a.name for a in self.arrays]
@@ -138,13 +142,14 @@ class PagedSpec:
 
 
 def kv_spec(kv_heads: int, head_dim: int, window: Optional[int] = None, v_transposed: bool = False,
-            value_dim: Optional[int] = None, chunk: Optional[int] = None) -> PagedSpec:
+            value_dim: Optional[int] = None, chunk: Optional[int] = None, keep_first: int = 0) -> PagedSpec:
     """Keys and values of grouped-query attention: K [kv_heads, page, head_dim]
     and V the same (value_dim wide where values have a size of their own), or
     transposed inside the page [kv_heads, value_dim, page]."""
     value_dim = head_dim if value_dim is None else value_dim
     v_shape = (kv_heads, value_dim, PAGE) if v_transposed else (kv_heads, PAGE, value_dim)
-    return PagedSpec((PagedArray("k", (kv_heads, PAGE, head_dim)), PagedArray("v", v_shape)), window, chunk=chunk)
+    return PagedSpec((PagedArray("k", (kv_heads, PAGE, head_dim)), PagedArray("v", v_shape)), window, chunk=chunk,
+                     keep_first=keep_first)
 
 
 @dataclass(frozen=True)
@@ -206,7 +211,7 @@ def with_fixed_arrays(spec: StateSpec, arrays: Sequence[FixedArray]) -> StateSpe
     old = fixed_part(spec)
     both = FixedSpec(arrays=(old.all_arrays() if old is not None else ()) + arrays)
     if isinstance(spec, PagedSpec):
-        return PagedSpec(spec.arrays, spec.window, both, spec.chunk)
+        return replace(spec, fixed=both)
     return both
 
 
@@ -251,7 +256,8 @@ class CacheGroup:
         self.tables = _Tables(manager, index)
 
     def first_needed_page(self, next_position: int) -> int:
-        """The lowest logical page a query at `next_position` or later reads."""
+        """The lowest logical page a query at `next_position` or later reads (beside the pages of the
+        first positions, where the group keeps those)."""
         return self._m._lib.imparo_cache_first_needed_page(self._m._c, self.index, next_position)
 
 
@@ -325,6 +331,8 @@ class CacheManager:
         self._c = self._lib.imparo_cache_new(len(specs), windows, page_size, pool_sizes, n_slots)
         if not self._c:
             raise ValueError("the cache manager refused its sizes")
+        for g, spec in enumerate(specs):
+            self._lib.imparo_cache_keep_first(self._c, g, spec.keep_first)
         self.groups: List[CacheGroup] = []
         for g, spec in enumerate(specs):
             pool = PagePool(0, _borrowed=self._lib.imparo_cache_group_pool(self._c, g))

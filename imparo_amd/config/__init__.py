@@ -22,3 +22,7 @@ from . import mepapel as _mepapel
 from .mepapel import MepapelConfig
 
 register_architecture(_mepapel.ARCHITECTURE, MepapelConfig.from_dict, _mepapel.build_plan)
+from . import vebusun as _vebusun
+from .vebusun import VebusunConfig
+
+register_architecture(_vebusun.ARCHITECTURE, VebusunConfig.from_dict, _vebusun.build_plan)

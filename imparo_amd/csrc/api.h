@@ -11,6 +11,22 @@ extern "C" {
 
 typedef void* imparo_stream;
 
+// What a layer's attention may ask for beyond a window. keep_first: the first so many positions stay visible to
+// every later query, whatever the window (a window of 0 sees everything anyway). softcap > 0: a scaled score s
+// becomes softcap * tanh(s / softcap). sink [heads] float32 or null: the softmax's denominator holds one more
+// term, exp(sink) of the head, which has no key and no value and is neither scaled nor capped. out_scale
+// multiplies the result in float32 before it is rounded.
+typedef struct {
+    int keep_first;
+    float softcap;
+    const float* sink;
+    float out_scale;
+} ImparoAttentionRule;
+static inline int imparo_attention_rule_bad(ImparoAttentionRule r, int window) {
+    return r.keep_first < 0 || !(r.softcap >= 0.f) || r.out_scale != r.out_scale || window < -(1 << 30) || window > (1 << 30) ||
+           r.keep_first > (1 << 30);
+}
+
 // The hash of the sources this library was built from, as the build computed it.
 const char* imparo_hip_source_hash();
 
@@ -37,6 +53,13 @@ int imparo_rms_norm(float* x, const float* delta, int n_delta, int n_x_rows, con
                     void* out, int out_dtype, int n_rows, int width, float eps, int write_back,
                     imparo_stream stream);
 
+// A norm without a statistic, row-wise: out[i, :] = tanh(alpha v) * weight + bias with v the source row rows[i] (or
+// i) of x plus the slices of up to two deltas (each [n, n_x_rows, width], added in order: first the slices of a
+// delta to one another, then the deltas to x). write_back (rows null): v is stored to x.
+int imparo_dynamic_tanh(float* x, const float* delta_a, int n_a, const float* delta_b, int n_b, int n_x_rows,
+                        const int32_t* rows, float alpha, const float* weight, const float* bias, void* out,
+                        int out_dtype, int n_rows, int width, int write_back, imparo_stream stream);
+
 // Y[m, n] = X[m, k] . W[n, k]^T (+ bias[n], float32, may be null), float32
 // accumulate. X and W share `dtype`. epilogue 0: Y is [m, n]. epilogue 1
 // (SwiGLU): W's rows alternate gate, up; Y is [m, n/2] with
@@ -46,6 +69,9 @@ int imparo_rms_norm(float* x, const float* delta, int n_delta, int n_x_rows, con
 // in slice 0); the consumer adds the slices in order.
 int imparo_gemm(const void* x, const void* w, const float* bias, void* y, int dtype, int out_dtype,
                 int m, int n, int k, int epilogue, int slices, imparo_stream stream);
+// epilogue 1 with the result multiplied by `scale` before it is rounded, one slice.
+int imparo_gemm_swiglu_scaled(const void* x, const void* w, const float* bias, void* y, int dtype, int out_dtype,
+                              int m, int n, int k, float scale, imparo_stream stream);
 int imparo_gemm_slices(int m, int n, int k, int dtype);
 // epilogue 2 (float32 out, `slices` 1): Y[m, n] += the product (+ bias), each element of Y read where it
 // is stored. Only for shapes for which imparo_gemm_adds gives 1 (many rows, a K the tile kernel takes).
@@ -98,6 +124,27 @@ int imparo_attention_prefill_exact(const void* q, const void* k_cache, const voi
                                    const int32_t* block_table, int table_stride, int page_size,
                                    int heads, int kv_heads, int head_dim, int n_pages, float scale, int window,
                                    imparo_stream stream);
+// The exact forms of decode and prefill for a layer with more rules than a window, and the most keys such a query
+// walks over at positions below max_context (the splits of a decode launch are counted from it). The wave kernel
+// likewise.
+int imparo_attention_ruled_keys(int max_context, int window, int keep_first);
+int imparo_attention_decode_ruled(const void* q, const void* k_cache, const void* v_cache, void* out, float* part_o,
+                                  float* part_ml, const int32_t* rows, int n_rows, const int32_t* seg_start,
+                                  const int32_t* positions, const int32_t* block_table, int table_stride, int page_size,
+                                  int heads, int kv_heads, int head_dim, int n_pages, float scale, int window,
+                                  int n_splits, const ImparoAttentionRule* rule, imparo_stream stream);
+int imparo_attention_prefill_ruled(const void* q, const void* k_cache, const void* v_cache, void* out, float* part_o,
+                                   float* part_ml, int n_splits, const int32_t* rows, int n_rows, int n_tiles,
+                                   const int32_t* seg_start, const int32_t* seg_len, const int32_t* positions,
+                                   const int32_t* block_table, int table_stride, int page_size, int heads, int kv_heads,
+                                   int head_dim, int n_pages, float scale, int window, const ImparoAttentionRule* rule,
+                                   imparo_stream stream);
+int imparo_attention_ruled(const void* q, const void* k_cache, const void* v_cache, void* out, int dtype,
+                           const int32_t* positions, const int32_t* row_of_token, const int32_t* block_table,
+                           int table_stride, int page_size, int n_tokens, int heads, int kv_heads, int head_dim,
+                           int value_dim, int out_ld, int n_pages, float scale, int window, int v_transposed,
+                           const ImparoAttentionRule* rule, imparo_stream stream);
+
 
 // The two above for heads whose values have another size than their keys (value_dim): a token's row is
 // heads + kv_heads units of head_dim, then kv_heads units of value_dim; the value cache holds value_dim a
@@ -191,17 +238,32 @@ int imparo_decay_scan(const float* q, int q_ld, int q_off, int q_div, const floa
                       int step_off, const float* step_bias, const float* rate, int v_times_step, const float* beta,
                       int beta_ld, int beta_off, const float* skip, float* state, const int32_t* seg_start,
                       const int32_t* seg_len, const int32_t* slot, float* out, int n_rows, int heads, int dim, int vdim,
-                      int chunk_tokens, int max_chunks, float* chunk_state, float* chunk_decay, imparo_stream stream);
+                      int chunk_tokens, int max_chunks, float* chunk_state, float* chunk_decay, int silu_in,
+                      imparo_stream stream);       // silu_in: q, k and v go through SiLU as they are read (chunk_tokens 0, no beta)
+// The gated delta rule with one decay a head and state row: S <- diag(g) S, u = b (v - S^T k), S <- S + k u^T,
+// o = S^T q with g = exp(-rate_h softplus(step[t, h dim + i] + bias[h dim + i])). chunk_tokens 0: token by token;
+// imparo_delta_chunk_tokens(): in chunks, dim at most imparo_delta_chunk_max_dim(), `scratch` holding n_rows *
+// max_chunks * heads * imparo_channel_delta_scratch(dim) floats.
+int imparo_channel_delta_scan(const float* q, int q_ld, int q_off, int q_div, const float* k, int k_ld, int k_off,
+                              int k_div, const float* v, int v_ld, int v_off, const float* step, int step_ld,
+                              int step_off, const float* step_bias, const float* rate, const float* beta, int beta_ld,
+                              int beta_off, float* state, const int32_t* seg_start, const int32_t* seg_len,
+                              const int32_t* slot, float* out, int n_rows, int heads, int dim, int vdim,
+                              int chunk_tokens, int max_chunks, float* scratch, imparo_stream stream);
+long long imparo_channel_delta_scratch(int dim);
+// Columns off .. off + n - 1 of float32 rows become their own SiLU.
+int imparo_silu_columns(float* rows, int ld, int off, int n, int n_tokens, imparo_stream stream);
 // Heads of `dim` columns from `off` on in float32 rows, in place: divided by sqrt(sum of squares + unit_eps) if
 // `unit`, the first 2 n_freq dimensions rotated by position (pairs (i, i + n_freq), or neighbours if interleaved),
 // multiplied by scale_first (heads below n_first) or scale_rest.
 int imparo_head_prepare(float* rows, int ld, int off, int n_tokens, int heads, int dim, int unit, float unit_eps,
                         const float* inv_freq, int n_freq, int interleaved, const int32_t* positions, int n_first,
                         float scale_first, float scale_rest, imparo_stream stream);
-// A row of `width` float32 values in `groups` equal parts, with g = silu(gate[t, gate_off + c]) (gate null: 1):
+// A row of `width` float32 values in `groups` equal parts, with g = silu(gate[t, gate_off + c]), or its sigmoid with
+// gate_act 1 (gate null: 1):
 // gate_first: (x g) / rms_part(x g) * w; otherwise x / rms_part(x) * w * g (w null: 1).
 int imparo_gated_group_norm(const float* x, const float* gate, int gate_ld, int gate_off, const float* w, void* out,
-                            int out_dtype, int n_tokens, int width, int groups, float eps, int gate_first,
+                            int out_dtype, int n_tokens, int width, int groups, float eps, int gate_first, int gate_act,
                             imparo_stream stream);
 // out[t, j] = g sigmoid(alpha g) (u + 1), g = min(gu[t, j], limit), u = clamp(gu[t, hidden + j], -limit, limit);
 // columns from `hidden` to out_ld are zero.

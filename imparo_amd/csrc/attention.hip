@@ -60,7 +60,7 @@ __global__ void k_attention_wave(const T* __restrict__ q, const T* __restrict__ 
                                  const int32_t* __restrict__ row_of_token, const int32_t* __restrict__ block_table,
                                  int table_stride, int page_size, int n_tokens, int heads, int kv_heads, int head_dim,
                                  int value_dim, int out_ld, int n_pages, float scale, int window, int v_transposed,
-                                 int v_ld) {
+                                 int v_ld, const ImparoAttentionRule rule) {
     __shared__ float q_rows[ATT_WAVES][ATT_MAX_HEAD_DIM];
     __shared__ float probs[ATT_WAVES][WAVE];
     __shared__ long long v_off[ATT_WAVES][WAVE];
@@ -86,9 +86,12 @@ __global__ void k_attention_wave(const T* __restrict__ q, const T* __restrict__ 
     for (int j = 0; j < DPL; ++j) acc[j] = 0.f;
     float m = -INFINITY, l = 0.f;
 
-    for (int c = (lo / WAVE) * WAVE; c <= pos; c += WAVE) {
+    // the first positions that stay visible come first, then the window: chunks between the two are skipped
+    const int lo_chunk = (lo / WAVE) * WAVE;
+    const int keep = rule.keep_first;
+    for (int c = keep > 0 ? 0 : lo_chunk; c <= pos; c = (c + WAVE >= keep && c + WAVE < lo_chunk) ? lo_chunk : c + WAVE) {
         const int p = c + lane;
-        const bool valid = p >= lo && p <= pos;
+        const bool valid = p <= pos && (p >= lo || p < keep);
         float s = -INFINITY;
         long long off = -1;
         if (valid) {
@@ -97,6 +100,7 @@ __global__ void k_attention_wave(const T* __restrict__ q, const T* __restrict__ 
                 off = (((long long)page * kv_heads + kvh) * page_size + (p % page_size)) * head_dim;
                 s = (head_dim % Vec16<T>::N == 0 ? dot_row<T>(qr, k_cache + off, head_dim)
                                                  : dot_row_any<T>(qr, k_cache + off, head_dim)) * scale;
+                if (rule.softcap > 0.f) s = rule.softcap * tanhf(s / rule.softcap);
                 // from here on `off` is where the key's value row starts
                 off = v_transposed ? ((long long)page * kv_heads + kvh) * page_size * value_dim + (p % page_size)
                                    : (((long long)page * kv_heads + kvh) * page_size + (p % page_size)) * v_ld;
@@ -126,7 +130,13 @@ __global__ void k_attention_wave(const T* __restrict__ q, const T* __restrict__ 
         }
         wave_lds_sync();
     }
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float inv = l > 0.f ? 1.0f / l : 0.f;
+    if (rule.sink) {                        // one more term of the denominator, without a key or a value
+        const float sink = rule.sink[h], top = fmaxf(m, sink);
+        const float w = (m == -INFINITY) ? 0.f : expf(m - top);
+        inv = w / fmaf(l, w, expf(sink - top));
+    }
+    inv *= rule.out_scale;
     T* dst = out + (size_t)t * out_ld + (size_t)h * value_dim;
 #pragma unroll
     for (int j = 0; j < DPL; ++j) {
@@ -156,12 +166,15 @@ static int attention_wave(const void* q, const void* k_cache, const void* v_cach
                           const int32_t* positions, const int32_t* row_of_token,
                           const int32_t* block_table, int table_stride, int page_size,
                           int n_tokens, int heads, int kv_heads, int head_dim, int value_dim, int out_ld,
-                          int n_pages, float scale, int window, int v_transposed, int v_ld, imparo_stream stream) {
+                          int n_pages, float scale, int window, int v_transposed, int v_ld, imparo_stream stream,
+                          const ImparoAttentionRule* rule = nullptr) {
     const int bad = check_attention_args(q, k_cache, v_cache, out, positions, row_of_token, block_table, table_stride,
                                          page_size, n_tokens, heads, kv_heads, head_dim, n_pages, window);
     if (bad) return bad;
     if (value_dim <= 0 || value_dim > ATT_MAX_HEAD_DIM || out_ld < heads * value_dim) return IMPARO_BAD_ARGUMENT;
     if (v_ld < value_dim || (v_transposed && v_ld != value_dim)) return IMPARO_BAD_ARGUMENT;
+    const ImparoAttentionRule r = rule ? *rule : ImparoAttentionRule{0, 0.f, nullptr, 1.0f};
+    if (imparo_attention_rule_bad(r, window)) return IMPARO_BAD_ARGUMENT;
     if (n_tokens == 0) return IMPARO_OK;
     const long long total = (long long)n_tokens * heads;
     const unsigned blocks = (unsigned)((total + ATT_WAVES - 1) / ATT_WAVES);
@@ -170,12 +183,12 @@ static int attention_wave(const void* q, const void* k_cache, const void* v_cach
         k_attention_wave<float><<<blocks, ATT_WAVES * WAVE, 0, s>>>(
             (const float*)q, (const float*)k_cache, (const float*)v_cache, (float*)out, positions, row_of_token,
             block_table, table_stride, page_size, n_tokens, heads, kv_heads, head_dim, value_dim, out_ld, n_pages, scale, window, v_transposed,
-            v_ld);
+            v_ld, r);
     else if (dtype == IMPARO_BF16)
         k_attention_wave<bf16_t><<<blocks, ATT_WAVES * WAVE, 0, s>>>(
             (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, positions, row_of_token,
             block_table, table_stride, page_size, n_tokens, heads, kv_heads, head_dim, value_dim, out_ld, n_pages, scale, window,
-            v_transposed, v_ld);
+            v_transposed, v_ld, r);
     else
         return IMPARO_BAD_ARGUMENT;
     return launch_status();
@@ -189,6 +202,16 @@ extern "C" int imparo_attention_dv(const void* q, const void* k_cache, const voi
     return attention_wave(q, k_cache, v_cache, out, dtype, positions, row_of_token, block_table, table_stride, page_size,
                           n_tokens, heads, kv_heads, head_dim, value_dim, out_ld, n_pages, scale, window, v_transposed,
                           value_dim, stream);
+}
+
+extern "C" int imparo_attention_ruled(const void* q, const void* k_cache, const void* v_cache, void* out, int dtype,
+                                      const int32_t* positions, const int32_t* row_of_token, const int32_t* block_table,
+                                      int table_stride, int page_size, int n_tokens, int heads, int kv_heads, int head_dim,
+                                      int value_dim, int out_ld, int n_pages, float scale, int window, int v_transposed,
+                                      const ImparoAttentionRule* rule, imparo_stream stream) {
+    return attention_wave(q, k_cache, v_cache, out, dtype, positions, row_of_token, block_table, table_stride, page_size,
+                          n_tokens, heads, kv_heads, head_dim, value_dim, out_ld, n_pages, scale, window, v_transposed,
+                          value_dim, stream, rule);
 }
 
 // Attention over a cached latent: every head reads the same rows [pages, page, row_dim]; a key is a whole

@@ -89,6 +89,45 @@ __device__ __forceinline__ uint4 zero_unless(bool keep, uint4 v) {
     return make_uint4(keep ? v.x : 0u, keep ? v.y : 0u, keep ? v.z : 0u, keep ? v.w : 0u);
 }
 
+// What a layer may ask for beyond a window (ImparoAttentionRule), where the kernels are built with EXT:
+// the first `keep` positions stay visible, scores go through cap * tanh(score / cap), the denominator holds one
+// more term exp(sink) of the head, and the result is multiplied by a constant before it is rounded.
+struct Rule {
+    int keep;
+    float cap;                  // 0: none
+    const float* sink;          // [heads] or null
+    float out_scale;
+};
+
+// tanh by the hardware's exp2 and reciprocal: within 2e-7 of it, and +-1 at both ends
+__device__ __forceinline__ float tanh_fast(float x) {
+    return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.88539008177792681472f * x));
+}
+
+// What a finished sum of weights `l` (relative to the maximum `m` of the scores) makes of the accumulated values:
+// the factor they are multiplied by.
+__device__ __forceinline__ float ruled_inverse(const Rule& rule, int head, float m, float l) {
+    float inv = l > 0.f ? 1.0f / l : 0.f;
+    if (rule.sink) {
+        const float sink = rule.sink[head], top = fmaxf(m, sink);
+        const float w = (m == -INFINITY) ? 0.f : __expf(m - top);
+        inv = w / fmaf(l, w, __expf(sink - top));
+    }
+    return inv * rule.out_scale;
+}
+
+// The tiles of TILE keys that a run of queries reads, numbered without the gap between the first positions that
+// stay and the window: tile base b of that numbering stands for key b, or b + gap once the kept tiles are passed.
+template <int TILE>
+struct TileWalk {
+    int keep_end, gap;
+    __device__ __forceinline__ TileWalk(int keep, int lo) {
+        keep_end = (keep + TILE - 1) & ~(TILE - 1);
+        gap = max(0, (lo & ~(TILE - 1)) - keep_end);
+    }
+    __device__ __forceinline__ int key(int base) const { return base < keep_end ? base : base + gap; }
+};
+
 // Issues the loads of the tile starting at key_base (a multiple of 32). [lo_all, hi_all] are
 // the live keys any query of the wave may read: addresses are clamped into it (what lies
 // outside is forced to zero before use). No load sits under a branch.
@@ -121,7 +160,7 @@ __device__ __forceinline__ void decode_load(DecodeTile<ND>& r, const Paged& kv, 
 template <int ND>
 __device__ __forceinline__ void decode_tile(DecodeState<ND>& st, const DecodeTile<ND>& r, int key_base, int lo_q,
                                             int hi_q, int lo_all, int hi_all, bool full, float scale, int lane,
-                                            bool exact = false) {
+                                            bool exact = false, int keep = 0, float cap = 0.f) {
     constexpr int D = ND * 16, NK = (ND + 1) / 2;
     const int g = lane >> 4;
     // ---- scores of keys kg .. kg+7: sv[4*t + i] from product t, row 4*g + i
@@ -141,8 +180,10 @@ __device__ __forceinline__ void decode_tile(DecodeState<ND>& st, const DecodeTil
     float mx = -INFINITY;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-        const bool ok = full || (kg + j >= lo_q && kg + j <= hi_q);
-        sv[j] = ok ? s[j >> 2][j & 3] * scale : -INFINITY;
+        const bool ok = full || ((kg + j >= lo_q || kg + j < keep) && kg + j <= hi_q);
+        float score = s[j >> 2][j & 3] * scale;
+        if (cap > 0.f) score = cap * tanh_fast(score * __builtin_amdgcn_rcpf(cap));
+        sv[j] = ok ? score : -INFINITY;
         mx = fmaxf(mx, sv[j]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
@@ -181,7 +222,7 @@ __device__ __forceinline__ void decode_tile(DecodeState<ND>& st, const DecodeTil
         if (!full) {
 #pragma unroll
             for (int j = 0; j < 8; ++j)
-                if (kg + j < lo_all || kg + j > hi_all) a.h[j] = 0;   // stale or foreign memory: never multiplied
+                if ((kg + j < lo_all && kg + j >= keep) || kg + j > hi_all) a.h[j] = 0;   // stale or foreign memory: never multiplied
         }
         st.o[dt] = st.o[dt] * corr;
         st.o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, pb.v, st.o[dt], 0, 0, 0);
@@ -285,13 +326,13 @@ __device__ __forceinline__ void normed_rotated(Frag8 (&out)[(ND + 1) / 2], HeadE
     }
 }
 
-template <int ND, bool FROM_QKV>
+template <int ND, bool FROM_QKV, bool EXT = false>
 __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 4 : 2) void k_attn_decode(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     float* __restrict__ part_o, float* __restrict__ part_ml, bf16_t* __restrict__ out,
     const int32_t* __restrict__ rows, const int32_t* __restrict__ seg_start, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ block_table, int table_stride, int page_size, int heads, int kv_heads, int n_pages,
-    float scale, int window, int n_splits, FromQkv fq, int exact) {
+    float scale, int window, int n_splits, FromQkv fq, int exact, Rule rule) {
     constexpr int D = ND * 16, NK = (ND + 1) / 2;
     constexpr int TILES = DEC_SPLIT / (MFMA_WAVES * 32);   // tiles a wave takes at most
     __shared__ float sm[MFMA_WAVES][16], sl[MFMA_WAVES][16];
@@ -307,8 +348,12 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 4 : 2) void k_attn_decod
     const int pos = positions[t];
     const int lo = first_seen(pos, window);
     const int last = FROM_QKV ? pos - 1 : pos;              // the last key that is in the cache
-    const int k_begin = max(split * DEC_SPLIT, lo & ~31);
-    const int k_end = min((split + 1) * DEC_SPLIT, last + 1);
+    // (EXT: splits count keys in the numbering without the gap behind the first positions that stay)
+    const TileWalk<32> walk(EXT ? rule.keep : 0, EXT ? lo : 0);
+    const int keep = EXT ? rule.keep : 0;
+    const float cap = EXT ? rule.cap : 0.f;
+    const int k_begin = EXT ? split * DEC_SPLIT : max(split * DEC_SPLIT, lo & ~31);
+    const int k_end = min((split + 1) * DEC_SPLIT, last + 1 - walk.gap);
     const bool own = FROM_QKV && split == pos / DEC_SPLIT;  // this block weighs the row's own key in
     if (k_begin >= k_end && !own) return;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -325,11 +370,11 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 4 : 2) void k_attn_decod
              __ffs(page_size) - 1};
     const int hi_q = qvalid ? last : -1;
     // (a block with the row's own key only: one clamped tile is loaded and none is used)
-    const int lo_c = min(lo, max(last, 0)), last_c = max(last, 0);
+    const int lo_c = (EXT && keep > 0) ? 0 : min(lo, max(last, 0)), last_c = max(last, 0);
     DecodeTile<ND> regs[TILES];
 #pragma unroll
     for (int j = 0; j < TILES; ++j)             // past the split's end: clamped addresses, never used
-        decode_load<ND>(regs[j], kv, k_begin + (wave + j * MFMA_WAVES) * 32, lo_c, last_c, lane);
+        decode_load<ND>(regs[j], kv, walk.key(k_begin + (wave + j * MFMA_WAVES) * 32), lo_c, last_c, lane);
     if (!FROM_QKV) {
         const bf16_t* qrow = q + ((size_t)t * heads + head) * D;
 #pragma unroll
@@ -362,10 +407,11 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 4 : 2) void k_attn_decod
     }
 #pragma unroll
     for (int j = 0; j < TILES; ++j) {
-        const int kb = k_begin + (wave + j * MFMA_WAVES) * 32;
-        if (kb < k_end) {
-            const bool full = kb >= lo && kb + 31 <= last;
-            decode_tile<ND>(st, regs[j], kb, lo, hi_q, lo, last, full, scale, lane, exact != 0);
+        const int kv_base = k_begin + (wave + j * MFMA_WAVES) * 32;
+        if (kv_base < k_end) {
+            const int kb = walk.key(kv_base);
+            const bool full = (kb >= lo || kb + 31 < keep) && kb + 31 <= last;
+            decode_tile<ND>(st, regs[j], kb, lo, hi_q, lo, last, full, scale, lane, exact != 0, keep, cap);
         }
     }
     if constexpr (FROM_QKV) {
@@ -444,7 +490,8 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 4 : 2) void k_attn_decod
         }
         const int head_out = kvh * G + pass * 16 + qc;
         if (n_splits == 1) {
-            out[((size_t)t * heads + head_out) * D + d] = f32_to_bf16(ls > 0.f ? acc / ls : 0.f);
+            const float o = EXT ? acc * ruled_inverse(rule, head_out, ms, ls) : (ls > 0.f ? acc / ls : 0.f);
+            out[((size_t)t * heads + head_out) * D + d] = f32_to_bf16(o);
             continue;
         }
         const size_t slot = ((size_t)ri * heads + head_out) * n_splits + split;
@@ -461,10 +508,11 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 4 : 2) void k_attn_decod
 // known after one round trip; the partial outputs then come eight splits at a
 // time, all loads of a group issued before the first is used, and are added in
 // split order.
+template <bool EXT>
 __global__ void k_attn_decode_merge(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                     bf16_t* __restrict__ out, const int32_t* __restrict__ rows,
                                     const int32_t* __restrict__ seg_start, const int32_t* __restrict__ positions,
-                                    int heads, int head_dim, int n_splits, int window) {
+                                    int heads, int head_dim, int n_splits, int window, Rule rule) {
     // A lane holds four neighbouring elements of the head, head_dim / 4 lanes a split's output, so the wave
     // takes several splits side by side (4 at head size 64), each lane GROUP of its splits' loads in flight at
     // once: a wave that fetches split after split makes one trip to memory after the other, and at 128 splits
@@ -478,7 +526,8 @@ __global__ void k_attn_decode_merge(const float* __restrict__ part_o, const floa
     const int t = seg_start[rows[ri]];
     const int pos = positions[t];
     const int lo = first_seen(pos, window);
-    const int s_lo = (lo & ~15) / DEC_SPLIT, s_hi = pos / DEC_SPLIT;
+    const int s_lo = EXT ? 0 : (lo & ~15) / DEC_SPLIT;
+    const int s_hi = (EXT ? pos - TileWalk<32>(rule.keep, lo).gap : pos) / DEC_SPLIT;
     const size_t base = ((size_t)ri * heads + head) * n_splits;
     float ms = -INFINITY;
     for (int s0 = s_lo; s0 <= s_hi; s0 += WAVE) {
@@ -525,7 +574,7 @@ __global__ void k_attn_decode_merge(const float* __restrict__ part_o, const floa
         for (int c = 0; c < 4; ++c) total[c] += __shfl(acc[c], (lane % lanes_a_split) + k * lanes_a_split, WAVE);
     }
     if (sub != 0) return;
-    const float inv = ls > 0.f ? 1.0f / ls : 0.f;
+    const float inv = EXT ? ruled_inverse(rule, head, ms, ls) : (ls > 0.f ? 1.0f / ls : 0.f);
     uint2 packed;
     packed.x = f32x2_to_bf16x2(total[0] * inv, total[1] * inv);
     packed.y = f32x2_to_bf16x2(total[2] * inv, total[3] * inv);
@@ -560,15 +609,16 @@ __device__ __forceinline__ void snake_block(int& tile, int& by) {
     tile = linear - by * gx;
 }
 
-template <int ND>
+template <int ND, bool EXT>
 __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     bf16_t* __restrict__ out, const int32_t* __restrict__ rows, int n_rows,
     const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_len, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ block_table, int table_stride, int page_size, int heads, int kv_heads, int n_pages,
-    float scale, int window, int exact) {
+    float scale, int window, int exact, Rule rule) {
     constexpr int D = ND * 16;
     constexpr int LDK = PF_LD_K(D);
+    const int keep = EXT ? rule.keep : 0;
     const int page_shift = __ffs(page_size) - 1;          // a power of two: divisions by it are shifts
     __shared__ __attribute__((aligned(16))) bf16_t ks[2][PF_KEYS * LDK];
     __shared__ __attribute__((aligned(16))) bf16_t vs[2][D * PF_LD_V];
@@ -613,7 +663,11 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
     const int lo_max = first_seen(pos_last, window);
     WaveState<ND> st;
     load_q<ND>(st, q + ((size_t)(t0 + min(qi, len - 1)) * heads + head) * D, qvalid && wave_on, lane);
-    const float scale_log2 = scale * 1.44269504088896340736f;
+    // capped scores are kept as tanh values, which the cap multiplies
+    const bool capped = EXT && rule.cap > 0.f;
+    const float in_cap = capped ? scale / rule.cap : 0.f;
+    const float scale_log2 = (capped ? rule.cap : scale) * 1.44269504088896340736f;
+    const TileWalk<PF_KEYS> walk(keep, EXT ? blk_lo : 0);
 
     // staging: K tile = 64 keys x D/8 pieces of 16 bytes; V^T tile = D rows x 8 pieces of 8 keys
     constexpr int K_PIECES = PF_KEYS * (D / 8), V_PIECES = D * (PF_KEYS / 8);
@@ -623,7 +677,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
 #pragma unroll
         for (int j = 0; j < K_PER; ++j) {
             const int p = tid + j * 256;
-            const int key = min(max(kb + p / (D / 8), blk_lo), blk_last);      // a live key: address always valid
+            const int key = min(max(kb + p / (D / 8), keep > 0 ? 0 : blk_lo), blk_last);   // the address is always valid
             int page = table[key >> page_shift];
             page = min(max(page, 0), n_pages - 1);
             kr[j] = (p < K_PIECES)
@@ -635,7 +689,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
         for (int j = 0; j < V_PER; ++j) {
             const int p = tid + j * 256;
             const int d = p / (PF_KEYS / 8), kg = kb + (p % (PF_KEYS / 8)) * 8;   // 8 keys kg .. kg+7, one page
-            const int kgc = min(max(kg, blk_lo & ~7), blk_last & ~7);
+            const int kgc = min(max(kg, keep > 0 ? 0 : blk_lo & ~7), blk_last & ~7);
             int page = table[kgc >> page_shift];
             page = min(max(page, 0), n_pages - 1);
             uint4 v = make_uint4(0, 0, 0, 0);
@@ -647,7 +701,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
                 uint32_t w[4] = {v.x, v.y, v.z, v.w};
 #pragma unroll
                 for (int e = 0; e < 8; ++e)
-                    if (kg + e < blk_lo || kg + e > blk_last) w[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
+                    if ((kg + e < blk_lo && kg + e >= keep) || kg + e > blk_last) w[e >> 1] &= (e & 1) ? 0x0000ffffu : 0xffff0000u;
                 v = make_uint4(w[0], w[1], w[2], w[3]);
             }
             vr[j] = v;
@@ -667,17 +721,17 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
         }
     };
 
-    const int kb_first = blk_lo & ~(PF_KEYS - 1);
+    const int kb_first = EXT ? walk.key(0) : blk_lo & ~(PF_KEYS - 1);
     stage_load(kb_first);
     stage_store(0);
     __syncthreads();
     int buf = 0;
-    for (int kb = kb_first; kb <= blk_last; kb += PF_KEYS) {
-        const int kn = kb + PF_KEYS;
+    for (int kb = kb_first; kb <= blk_last;) {
+        const int kn = EXT ? (kb + PF_KEYS == walk.keep_end ? kb + PF_KEYS + walk.gap : kb + PF_KEYS) : kb + PF_KEYS;
         if (kn <= blk_last) stage_load(kn);
-        // this wave's part of the tile: keys lo_all .. pos_last
-        if (wave_on && kb <= pos_last && kb + PF_KEYS - 1 >= lo_all) {
-            const bool full = kb >= lo_max && kb + PF_KEYS - 1 <= pos_first;
+        // this wave's part of the tile: keys lo_all .. pos_last, and those that stay
+        if (wave_on && kb <= pos_last && (kb + PF_KEYS - 1 >= lo_all || kb < keep)) {
+            const bool full = (kb >= lo_max || kb + PF_KEYS - 1 < keep) && kb + PF_KEYS - 1 <= pos_first;
             f32x4 sc[4];
 #pragma unroll
             for (int kt = 0; kt < 4; ++kt) {
@@ -688,6 +742,12 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
                     const s16x4 a = *reinterpret_cast<const s16x4*>(krow + dk * 16);
                     sc[kt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(a, st.q[dk], sc[kt], 0, 0, 0);
                 }
+            }
+            if (capped) {
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) sc[kt][i] = tanh_fast(sc[kt][i] * in_cap);
             }
             // sc[kt][i] = score of key kb + 16 kt + 4 g + i for query lane%16. The running maximum
             // st.m is kept in units of log2(e), so that every weight is one exp2 of a difference.
@@ -706,7 +766,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         const int kp = kb + kt * 16 + 4 * g + i;
-                        sc[kt][i] = (kp >= lo_q && kp <= hi_q) ? sc[kt][i] * scale_log2 : -INFINITY;
+                        sc[kt][i] = ((kp >= lo_q || kp < keep) && kp <= hi_q) ? sc[kt][i] * scale_log2 : -INFINITY;
                         mx = fmaxf(mx, sc[kt][i]);
                     }
             }
@@ -756,9 +816,10 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
         if (kn <= blk_last) stage_store(buf ^ 1);
         __syncthreads();
         buf ^= 1;
+        kb = kn;
     }
     if (!qvalid || !wave_on) return;
-    const float inv = st.l > 0.f ? 1.0f / st.l : 0.f;
+    const float inv = EXT ? ruled_inverse(rule, head, st.m * 0.69314718055994530942f, st.l) : (st.l > 0.f ? 1.0f / st.l : 0.f);
     bf16_t* dst = out + ((size_t)(t0 + qi) * heads + head) * D + 4 * g;
 #pragma unroll
     for (int dt = 0; dt < ND; ++dt) {
@@ -789,15 +850,16 @@ __global__ __launch_bounds__(MFMA_WAVES * 64) void k_attn_prefill(
 // block table a tile then serves every thread, and what a thread reads of a tile is at a fixed place
 // inside the page: a quarter of the instructions of the general staging, which was a quarter to a
 // third of the kernel's time.
-template <int ND, int HALVES, bool PAGE_TILE>
+template <int ND, int HALVES, bool PAGE_TILE, bool EXT>
 __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefill_x32(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     bf16_t* __restrict__ out, const int32_t* __restrict__ rows, int n_rows,
     const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_len, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ block_table, int table_stride, int page_size, int heads, int kv_heads, int n_pages,
     float scale, int window, int heads_per_block, float* __restrict__ part_o, float* __restrict__ part_ml,
-    int exact) {
+    int exact, Rule rule) {
     constexpr int D = ND * 16, NK = ND / 2;
+    const int keep = EXT ? rule.keep : 0;
     // Rows of K lie their length + 32 bytes apart: the fragment reads (row lane % 16, 16-byte piece lane / 16) then
     // meet no bank conflict at any head size (with 16 bytes of padding each read takes 8 cycles instead of 4; counted
     // with SQ_LDS_BANK_CONFLICT on reads alone). V^T rows keep 16 bytes: 32 would free its reads too but make the
@@ -839,14 +901,31 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
     int blk_last = pos0 + min(len, tile * qt + qt) - 1;
     int blk_lo = first_seen(blk_first, window);
     const int n_splits = (int)gridDim.z, split = (int)blockIdx.z;
-    if (n_splits > 1) {
+    // EXT: tiles are numbered without the gap between the first positions that stay and the window; the block
+    // takes tile bases w_first .. w_last of that numbering
+    const TileWalk<PX_KEYS> walk(keep, EXT ? blk_lo : 0);
+    int w_first = 0, w_last = blk_last - walk.gap;
+    bool has_keys = true;
+    if constexpr (EXT) {
+        if (n_splits > 1) {
+            const int per = (w_last / PX_KEYS + n_splits) / n_splits;        // of w_last / PX_KEYS + 1 tiles
+            w_first = split * per * PX_KEYS;
+            w_last = min(w_last, (split + 1) * per * PX_KEYS - 1);
+            has_keys = w_first <= w_last;
+            if (!has_keys) w_first = w_last = 0;             // one masked tile, a partial of zero weight
+        }
+    } else if (n_splits > 1) {
         const int first_tile = blk_lo / PX_KEYS, tiles_all = blk_last / PX_KEYS - first_tile + 1;
         const int per = (tiles_all + n_splits - 1) / n_splits;
         blk_lo = max(blk_lo, (first_tile + split * per) * PX_KEYS);
         blk_last = min(blk_last, (first_tile + (split + 1) * per) * PX_KEYS - 1);
     }
-    const bool has_keys = blk_lo <= blk_last;
-    if (!has_keys) blk_lo = blk_last = max(blk_first, 0);       // nothing to add: one masked tile, a partial of zero weight
+    if constexpr (!EXT) {
+        has_keys = blk_lo <= blk_last;
+        if (!has_keys) blk_lo = blk_last = max(blk_first, 0);   // nothing to add: one masked tile, a partial of zero weight
+        w_first = blk_lo & ~(PX_KEYS - 1);
+        w_last = blk_last;
+    }
 
     // this wave's queries: q_first + 16 h + c for the halves h
     const int q_first = tile * qt + (wave / heads_per_block) * QW;
@@ -883,7 +962,10 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
         m_run[h] = -INFINITY;
         l_acc[h] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    const float scale_log2 = scale * 1.44269504088896340736f;
+    // capped scores are kept as tanh values, which the cap multiplies
+    const bool capped = EXT && rule.cap > 0.f;
+    const float in_cap = capped ? scale / rule.cap : 0.f;
+    const float scale_log2 = (capped ? rule.cap : scale) * 1.44269504088896340736f;
 
     // Staging: K tile = 64 keys x D/8 pieces of 16 bytes; V^T tile = D rows x 8 pieces of 8 keys; with
     // head sizes in steps of 32 the 256 threads take a whole number of pieces each. A piece's
@@ -899,7 +981,8 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
     // (the compiler's own vector type: an array of HIP's uint4 stays in memory)
     u32x4 kr_a[K_PER], vr_a[V_PER], kr_b[K_PER], vr_b[V_PER];
     int kpage[K_PER], vpage[V_PER];
-    const int kb_last = blk_last & ~(PX_KEYS - 1);
+    const int kb_last = w_last & ~(PX_KEYS - 1);
+    const int lo_addr = (EXT && keep > 0) ? 0 : blk_lo;
     // PAGE_TILE: where in a page this thread's pieces of a tile lie that starts at the page's first position
     unsigned k_at[K_PER], v_at[V_PER];
 #pragma unroll
@@ -914,6 +997,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
     }
     auto load_pages = [&](int kb) __attribute__((always_inline)) {
         kb = min(kb, kb_last);
+        if constexpr (EXT) kb = walk.key(kb);
         if constexpr (PAGE_TILE) {
             kpage[0] = table[kb >> page_shift];       // the tile's page: it holds a live key, so it is there
             return;
@@ -921,18 +1005,19 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
 #pragma unroll
         for (int j = 0; j < K_PER; ++j) {
             const int pc = tid + j * 256;
-            const int key = min(max(kb + pc / (D / 8), blk_lo), blk_last);     // a live key: address always valid
+            const int key = min(max(kb + pc / (D / 8), lo_addr), blk_last);    // the address is always valid
             kpage[j] = table[key >> page_shift];
         }
 #pragma unroll
         for (int j = 0; j < V_PER; ++j) {
             const int pc = tid + j * 256;
-            const int kgc = min(max(kb + (pc % (PX_KEYS / 8)) * 8, blk_lo & ~7), blk_last & ~7);
+            const int kgc = min(max(kb + (pc % (PX_KEYS / 8)) * 8, lo_addr & ~7), blk_last & ~7);
             vpage[j] = table[kgc >> page_shift];
         }
     };
     auto load_data = [&](int kb, u32x4 (&kr)[K_PER], u32x4 (&vr)[V_PER]) __attribute__((always_inline)) {
         kb = min(kb, kb_last);
+        if constexpr (EXT) kb = walk.key(kb);
         if constexpr (PAGE_TILE) {
             // (keys of the page outside the live range are read too: what they hold is masked, and zeroed
             // where it would be multiplied)
@@ -947,7 +1032,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
 #pragma unroll
         for (int j = 0; j < K_PER; ++j) {
             const int pc = tid + j * 256;
-            const int key = min(max(kb + pc / (D / 8), blk_lo), blk_last);
+            const int key = min(max(kb + pc / (D / 8), lo_addr), blk_last);
             const int page = min(max(kpage[j], 0), n_pages - 1);
             const unsigned in_page = (unsigned)(kvh * page_size + (key & (page_size - 1))) * D + (pc % (D / 8)) * 8;
             kr[j] = *reinterpret_cast<const u32x4*>(k_cache + (size_t)page * page_elems + in_page);
@@ -956,7 +1041,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
         for (int j = 0; j < V_PER; ++j) {
             const int pc = tid + j * 256;
             const int d = pc / (PX_KEYS / 8);
-            const int kgc = min(max(kb + (pc % (PX_KEYS / 8)) * 8, blk_lo & ~7), blk_last & ~7);   // 8 keys, one page
+            const int kgc = min(max(kb + (pc % (PX_KEYS / 8)) * 8, lo_addr & ~7), blk_last & ~7);  // 8 keys, one page
             const int page = min(max(vpage[j], 0), n_pages - 1);
             const unsigned in_page = (unsigned)(kvh * D + d) * page_size + (kgc & (page_size - 1));
             vr[j] = *reinterpret_cast<const u32x4*>(v_cache + (size_t)page * page_elems + in_page);
@@ -964,6 +1049,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
     };
     // the tile whose data is in kr/vr goes to LDS: kb is its first key
     auto stage_store = [&](int kb, int buf, const u32x4 (&kr)[K_PER], const u32x4 (&vr)[V_PER]) __attribute__((always_inline)) {
+        if constexpr (EXT) kb = walk.key(kb);
 #pragma unroll
         for (int j = 0; j < K_PER; ++j) {
             const int pc = tid + j * 256;
@@ -980,7 +1066,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
             if (kb < blk_lo || kb + PX_KEYS - 1 > blk_last) {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) {
-                    const bool dead = kg + e < blk_lo || kg + e > blk_last;
+                    const bool dead = (kg + e < blk_lo && kg + e >= keep) || kg + e > blk_last;
                     w[e >> 1] = dead ? (w[e >> 1] & ((e & 1) ? 0x0000ffffu : 0xffff0000u)) : w[e >> 1];
                 }
             }
@@ -994,10 +1080,12 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
     // One tile: LDS buffer `buf` holds it and `have` the next tile's data, asked for two tiles ago, which goes
     // to the other LDS buffer once this tile is done; the set is then free and takes the loads of the tile
     // three further on (the other set holds the tile in between).
-    auto tile_step = [&](int kb, int buf, u32x4 (&kr_have)[K_PER], u32x4 (&vr_have)[V_PER]) __attribute__((always_inline)) {
-        // this wave's part of the tile: keys lo_all .. pos_last
-        if (wave_on && kb <= pos_last && kb + PX_KEYS - 1 >= lo_all) {
-            const bool full = kb >= lo_max && kb + PX_KEYS - 1 <= pos_first && kb >= blk_lo && kb + PX_KEYS - 1 <= blk_last;
+    auto tile_step = [&](int base, int buf, u32x4 (&kr_have)[K_PER], u32x4 (&vr_have)[V_PER]) __attribute__((always_inline)) {
+        const int kb = EXT ? walk.key(base) : base;
+        // this wave's part of the tile: keys lo_all .. pos_last, and those that stay
+        if (wave_on && kb <= pos_last && (kb + PX_KEYS - 1 >= lo_all || kb < keep)) {
+            const bool full = EXT ? (kb >= lo_max || kb + PX_KEYS - 1 < keep) && kb + PX_KEYS - 1 <= pos_first && has_keys
+                                  : kb >= lo_max && kb + PX_KEYS - 1 <= pos_first && kb >= blk_lo && kb + PX_KEYS - 1 <= blk_last;
             f32x4 sc[HALVES][4];
 #pragma unroll
             for (int s16 = 0; s16 < 4; ++s16) {
@@ -1012,6 +1100,14 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
                     for (int h = 0; h < HALVES; ++h)
                         sc[h][s16] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf.v, qf[h][dk].v, sc[h][s16], 0, 0, 0);
                 }
+            }
+            if (capped) {
+#pragma unroll
+                for (int h = 0; h < HALVES; ++h)
+#pragma unroll
+                    for (int s16 = 0; s16 < 4; ++s16)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) sc[h][s16][i] = tanh_fast(sc[h][s16][i] * in_cap);
             }
             // sc[h][s16][i] = score of key kb + 16 s16 + 4 g + i for query (h, lane%16), unscaled. The
             // running maximum is kept unscaled too: a weight is one fused multiply-add and one exp2,
@@ -1032,7 +1128,7 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
 #pragma unroll
                         for (int i = 0; i < 4; ++i) {
                             const int kp = kb + s16 * 16 + 4 * g + i;
-                            sc[h][s16][i] = (kp >= lo_q[h] && kp <= hi_q[h]) ? sc[h][s16][i] : -INFINITY;
+                            sc[h][s16][i] = ((kp >= lo_q[h] || kp < keep) && kp <= hi_q[h]) ? sc[h][s16][i] : -INFINITY;
                             mx = fmaxf(mx, sc[h][s16][i]);
                         }
                 }
@@ -1102,12 +1198,12 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
                 }
             }
         }
-        stage_store(min(kb + PX_KEYS, kb_last), buf ^ 1, kr_have, vr_have);
-        load_data(kb + 3 * PX_KEYS, kr_have, vr_have);      // with the pages asked for a tile ago
-        load_pages(kb + 4 * PX_KEYS);
+        stage_store(min(base + PX_KEYS, kb_last), buf ^ 1, kr_have, vr_have);
+        load_data(base + 3 * PX_KEYS, kr_have, vr_have);    // with the pages asked for a tile ago
+        load_pages(base + 4 * PX_KEYS);
         __syncthreads();
     };
-    const int kb_first = blk_lo & ~(PX_KEYS - 1);
+    const int kb_first = w_first;
     load_pages(kb_first);
     load_data(kb_first, kr_a, vr_a);
     load_pages(kb_first + PX_KEYS);
@@ -1117,9 +1213,9 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
     load_data(kb_first + 2 * PX_KEYS, kr_a, vr_a);
     load_pages(kb_first + 3 * PX_KEYS);
     __syncthreads();
-    for (int kb = kb_first; kb <= blk_last; kb += 2 * PX_KEYS) {
+    for (int kb = kb_first; kb <= w_last; kb += 2 * PX_KEYS) {
         tile_step(kb, 0, kr_b, vr_b);
-        if (kb + PX_KEYS > blk_last) break;
+        if (kb + PX_KEYS > w_last) break;
         tile_step(kb + PX_KEYS, 1, kr_a, vr_a);
     }
     if (!wave_on) return;
@@ -1142,7 +1238,8 @@ __global__ __launch_bounds__(MFMA_WAVES * 64, ND <= 4 ? 2 : 1) void k_attn_prefi
 #pragma unroll
     for (int h = 0; h < HALVES; ++h) {
         if (!qvalid[h]) continue;
-        const float inv = l_acc[h][0] > 0.f ? 1.0f / l_acc[h][0] : 0.f;
+        const float inv = EXT ? ruled_inverse(rule, head, m_run[h] * (capped ? rule.cap : scale), l_acc[h][0])
+                              : (l_acc[h][0] > 0.f ? 1.0f / l_acc[h][0] : 0.f);
         bf16_t* dst = out + ((size_t)(t0 + q_first + 16 * h + c) * heads + head) * D + 4 * g;
 #pragma unroll
         for (int dt = 0; dt < ND; ++dt) {
@@ -1164,8 +1261,9 @@ template <int GROUP>
 __global__ void k_attn_prefill_merge(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                      bf16_t* __restrict__ out, const int32_t* __restrict__ rows, int n_rows,
                                      const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_len,
-                                     int heads, int head_dim, int n_splits, float scale) {
+                                     int heads, int head_dim, int n_splits, float scale, Rule rule) {
     int tok = blockIdx.x, t = -1;
+    if (rule.cap > 0.f) scale = rule.cap;
     for (int i = 0; i < n_rows; ++i) {                   // the tok-th token of the listed rows
         const int r = rows[i];
         if (tok < seg_len[r]) {
@@ -1213,7 +1311,7 @@ __global__ void k_attn_prefill_merge(const float* __restrict__ part_o, const flo
             acc[3] += counts ? o[j].w * wgt : 0.f;
         }
     }
-    const float inv = ls > 0.f ? 1.0f / ls : 0.f;
+    const float inv = ruled_inverse(rule, head, ms * scale, ls);
     uint2 packed;
     packed.x = (uint32_t)f32_to_bf16(acc[0] * inv) | ((uint32_t)f32_to_bf16(acc[1] * inv) << 16);
     packed.y = (uint32_t)f32_to_bf16(acc[2] * inv) | ((uint32_t)f32_to_bf16(acc[3] * inv) << 16);
@@ -1252,13 +1350,20 @@ static int check_common(const void* q, const void* k_cache, const void* v_cache,
 extern "C" int imparo_attention_decode_split() { return DEC_SPLIT; }
 extern "C" int imparo_attention_prefill_tile() { return 64; }
 
+static Rule rule_of(const ImparoAttentionRule* r) {
+    return r ? Rule{r->keep_first, r->softcap, r->sink, r->out_scale} : Rule{0, 0.f, nullptr, 1.0f};
+}
+
 static int attention_decode_launch(const void* q, const void* k_cache, const void* v_cache, void* out,
                                    float* part_o, float* part_ml, const int32_t* rows, int n_rows,
                                    const int32_t* seg_start, const int32_t* positions,
                                    const int32_t* block_table, int table_stride, int page_size,
                                    int heads, int kv_heads, int head_dim, int n_pages, float scale, int window,
-                                   int n_splits, hipStream_t s, const FromQkv* from_qkv = nullptr, int exact = 0) {
+                                   int n_splits, hipStream_t s, const FromQkv* from_qkv = nullptr, int exact = 0,
+                                   const ImparoAttentionRule* given = nullptr) {
     const int G = heads / kv_heads;
+    const Rule rule = rule_of(given);
+    if (given && from_qkv) return IMPARO_BAD_ARGUMENT;
     // the merge moves four elements of a head in one access
     if (n_splits > 1 && (((uintptr_t)part_o & 15) || ((uintptr_t)out & 7))) return IMPARO_BAD_ARGUMENT;
     dim3 grid(n_splits, kv_heads * ((G + 15) / 16), n_rows);
@@ -1266,21 +1371,30 @@ static int attention_decode_launch(const void* q, const void* k_cache, const voi
 #define DECODE_FROM_QKV(ND)                                                                                          \
     k_attn_decode<ND, true><<<grid, MFMA_WAVES * 64, 0, s>>>(                                                        \
         nullptr, (const bf16_t*)k_cache, (const bf16_t*)v_cache, part_o, part_ml, (bf16_t*)out, rows, seg_start,     \
-        positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window, n_splits, *from_qkv, 0)
+        positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window, n_splits, *from_qkv, 0, rule)
         if (head_dim == 64) DECODE_FROM_QKV(4);
         else if (head_dim == 128) DECODE_FROM_QKV(8);
         else return IMPARO_BAD_ARGUMENT;
 #undef DECODE_FROM_QKV
+    } else if (given) {
+        DISPATCH_ND(head_dim / 16, (k_attn_decode<ND, false, true><<<grid, MFMA_WAVES * 64, 0, s>>>(
+            (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, part_o, part_ml, (bf16_t*)out, rows,
+            seg_start, positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window,
+            n_splits, FromQkv{}, exact, rule)));
     } else {
         DISPATCH_ND(head_dim / 16, (k_attn_decode<ND, false><<<grid, MFMA_WAVES * 64, 0, s>>>(
             (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, part_o, part_ml, (bf16_t*)out, rows,
             seg_start, positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window,
-            n_splits, FromQkv{}, exact)));
+            n_splits, FromQkv{}, exact, rule)));
     }
     if (launch_status()) return IMPARO_LAUNCH_FAILED;
     if (n_splits == 1) return IMPARO_OK;
-    k_attn_decode_merge<<<n_rows * heads, 64, 0, s>>>(part_o, part_ml, (bf16_t*)out, rows, seg_start, positions, heads,
-                                                      head_dim, n_splits, window);
+    if (given)
+        k_attn_decode_merge<true><<<n_rows * heads, 64, 0, s>>>(part_o, part_ml, (bf16_t*)out, rows, seg_start, positions,
+                                                                heads, head_dim, n_splits, window, rule);
+    else
+        k_attn_decode_merge<false><<<n_rows * heads, 64, 0, s>>>(part_o, part_ml, (bf16_t*)out, rows, seg_start, positions,
+                                                                 heads, head_dim, n_splits, window, rule);
     return launch_status();
 }
 
@@ -1289,7 +1403,9 @@ static int attention_decode_entry(const void* q, const void* k_cache, const void
                                   const int32_t* seg_start, const int32_t* positions,
                                   const int32_t* block_table, int table_stride, int page_size,
                                   int heads, int kv_heads, int head_dim, int n_pages, float scale, int window,
-                                  int n_splits, imparo_stream stream, int exact) {
+                                  int n_splits, imparo_stream stream, int exact,
+                                  const ImparoAttentionRule* rule = nullptr) {
+    if (rule && imparo_attention_rule_bad(*rule, window)) return IMPARO_BAD_ARGUMENT;
     const int bad = check_common(q, k_cache, v_cache, out, rows, seg_start, positions, block_table, table_stride,
                                  page_size, heads, kv_heads, head_dim, n_pages, window);
     if (bad) return bad;
@@ -1298,7 +1414,7 @@ static int attention_decode_entry(const void* q, const void* k_cache, const void
     if (n_rows > 65535) return IMPARO_BAD_ARGUMENT;
     return attention_decode_launch(q, k_cache, v_cache, out, part_o, part_ml, rows, n_rows, seg_start, positions,
                                    block_table, table_stride, page_size, heads, kv_heads, head_dim, n_pages, scale,
-                                   window, n_splits, (hipStream_t)stream, nullptr, exact);
+                                   window, n_splits, (hipStream_t)stream, nullptr, exact, rule);
 }
 
 extern "C" int imparo_attention_decode(const void* q, const void* k_cache, const void* v_cache, void* out,
@@ -1323,6 +1439,29 @@ extern "C" int imparo_attention_decode_exact(const void* q, const void* k_cache,
     return attention_decode_entry(q, k_cache, v_cache, out, part_o, part_ml, rows, n_rows, seg_start, positions,
                                   block_table, table_stride, page_size, heads, kv_heads, head_dim, n_pages, scale,
                                   window, n_splits, stream, 1);
+}
+
+// The exact form for a layer with more rules than a window (api.h: ImparoAttentionRule). The splits count the keys that
+// the row's query can see (n_splits = ceil of imparo_attention_ruled_keys / imparo_attention_decode_split()).
+extern "C" int imparo_attention_decode_ruled(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                             float* part_o, float* part_ml, const int32_t* rows, int n_rows,
+                                             const int32_t* seg_start, const int32_t* positions,
+                                             const int32_t* block_table, int table_stride, int page_size,
+                                             int heads, int kv_heads, int head_dim, int n_pages, float scale,
+                                             int window, int n_splits, const ImparoAttentionRule* rule,
+                                             imparo_stream stream) {
+    if (!rule) return IMPARO_BAD_ARGUMENT;
+    return attention_decode_entry(q, k_cache, v_cache, out, part_o, part_ml, rows, n_rows, seg_start, positions,
+                                  block_table, table_stride, page_size, heads, kv_heads, head_dim, n_pages, scale,
+                                  window, n_splits, stream, 1, rule);
+}
+
+// The most keys a query walks over under a window and first positions that stay, in tiles, at any position below
+// `max_context`: what the splits of such a launch are counted from. A chunk's length stands in for a window's.
+extern "C" int imparo_attention_ruled_keys(int max_context, int window, int keep_first) {
+    if (window == 0) return max_context;
+    const long long seen = (long long)(window > 0 ? window : -(long long)window) + 31 + (keep_first + 31LL) / 32 * 32;
+    return (int)std::min<long long>(max_context, seen);
 }
 
 // Which head sizes and rotations imparo_attention_decode_qkv takes: 64 or 128, rotated whole or not at all.
@@ -1479,7 +1618,9 @@ static int attention_prefill_entry(const void* q, const void* k_cache, const voi
                                    const int32_t* seg_start, const int32_t* seg_len, const int32_t* positions,
                                    const int32_t* block_table, int table_stride, int page_size,
                                    int heads, int kv_heads, int head_dim, int n_pages, float scale, int window,
-                                   imparo_stream stream, int exact) {
+                                   imparo_stream stream, int exact, const ImparoAttentionRule* given = nullptr) {
+    if (given && imparo_attention_rule_bad(*given, window)) return IMPARO_BAD_ARGUMENT;
+    const Rule rule = rule_of(given);
     const int bad = check_common(q, k_cache, v_cache, out, rows, seg_start, positions, block_table, table_stride,
                                  page_size, heads, kv_heads, head_dim, n_pages, window);
     if (bad) return bad;
@@ -1496,11 +1637,16 @@ static int attention_prefill_entry(const void* q, const void* k_cache, const voi
         const int hpb = p.hpb;
         const bool wide = p.wide;
         dim3 grid32((unsigned)(n_tiles * (p.qt < 64 ? 64 / p.qt : 1)), heads / hpb, n_splits);
-#define PREFILL_X32_GO(ND, HALVES, PAGE_TILE)                                                                       \
-    k_attn_prefill_x32<ND, HALVES, PAGE_TILE><<<grid32, MFMA_WAVES * 64, 0, s>>>(                                    \
+#define PREFILL_X32_RUN(ND, HALVES, PAGE_TILE, EXT)                                                                 \
+    k_attn_prefill_x32<ND, HALVES, PAGE_TILE, EXT><<<grid32, MFMA_WAVES * 64, 0, s>>>(                               \
         (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, rows, n_rows, seg_start,     \
         seg_len, positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window, hpb,      \
-        part_o, part_ml, exact)
+        part_o, part_ml, exact, rule)
+#define PREFILL_X32_GO(ND, HALVES, PAGE_TILE)                                                                       \
+    do {                                                                                                             \
+        if (given) PREFILL_X32_RUN(ND, HALVES, PAGE_TILE, true);                                                     \
+        else PREFILL_X32_RUN(ND, HALVES, PAGE_TILE, false);                                                          \
+    } while (0)
 #define PREFILL_X32(ND)                                                                                              \
     if (wide && page_size >= PX_KEYS) PREFILL_X32_GO(ND, 2, true);                                                   \
     else if (wide) PREFILL_X32_GO(ND, 2, false);                                                                     \
@@ -1514,6 +1660,7 @@ static int attention_prefill_entry(const void* q, const void* k_cache, const voi
         }
 #undef PREFILL_X32
 #undef PREFILL_X32_GO
+#undef PREFILL_X32_RUN
         if (launch_status()) return IMPARO_LAUNCH_FAILED;
         if (n_splits == 1) return IMPARO_OK;
         // a block of four waves per token, each wave as many heads as its lanes hold; tokens past the portions'
@@ -1522,7 +1669,7 @@ static int attention_prefill_entry(const void* q, const void* k_cache, const voi
         dim3 merge_grid((unsigned)n_tiles * 64, (unsigned)((heads + heads_a_block - 1) / heads_a_block));
 #define MERGE(GROUP)                                                                                              \
     k_attn_prefill_merge<GROUP><<<merge_grid, 256, 0, s>>>(part_o, part_ml, (bf16_t*)out, rows, n_rows, seg_start, \
-                                                           seg_len, heads, head_dim, n_splits, scale)
+                                                           seg_len, heads, head_dim, n_splits, scale, rule)
         if (n_splits <= 2) MERGE(2);
         else if (n_splits <= 4) MERGE(4);
         else MERGE(8);
@@ -1530,9 +1677,15 @@ static int attention_prefill_entry(const void* q, const void* k_cache, const voi
         return launch_status();
     }
     dim3 grid(n_tiles, heads);
-    DISPATCH_ND(head_dim / 16, (k_attn_prefill<ND><<<grid, MFMA_WAVES * 64, 0, s>>>(
+    if (given) {
+        DISPATCH_ND(head_dim / 16, (k_attn_prefill<ND, true><<<grid, MFMA_WAVES * 64, 0, s>>>(
+            (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, rows, n_rows, seg_start,
+            seg_len, positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window, exact, rule)));
+        return launch_status();
+    }
+    DISPATCH_ND(head_dim / 16, (k_attn_prefill<ND, false><<<grid, MFMA_WAVES * 64, 0, s>>>(
         (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, rows, n_rows, seg_start,
-        seg_len, positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window, exact)));
+        seg_len, positions, block_table, table_stride, page_size, heads, kv_heads, n_pages, scale, window, exact, rule)));
     return launch_status();
 }
 
@@ -1562,11 +1715,26 @@ extern "C" int imparo_attention_prefill_exact(const void* q, const void* k_cache
                                    n_pages, scale, window, stream, 1);
 }
 
+// The exact form for a layer with more rules than a window (api.h: ImparoAttentionRule).
+extern "C" int imparo_attention_prefill_ruled(const void* q, const void* k_cache, const void* v_cache, void* out,
+                                              float* part_o, float* part_ml, int n_splits,
+                                              const int32_t* rows, int n_rows, int n_tiles,
+                                              const int32_t* seg_start, const int32_t* seg_len,
+                                              const int32_t* positions, const int32_t* block_table, int table_stride,
+                                              int page_size, int heads, int kv_heads, int head_dim, int n_pages,
+                                              float scale, int window, const ImparoAttentionRule* rule,
+                                              imparo_stream stream) {
+    if (!rule) return IMPARO_BAD_ARGUMENT;
+    return attention_prefill_entry(q, k_cache, v_cache, out, part_o, part_ml, n_splits, rows, n_rows, n_tiles, seg_start,
+                                   seg_len, positions, block_table, table_stride, page_size, heads, kv_heads, head_dim,
+                                   n_pages, scale, window, stream, 1, rule);
+}
+
 // Asks the runtime about one kernel of this file, which makes it load the file's code onto the
 // current device (it loads a file's kernels when one of them is first used; a stream under capture
 // cannot do that).
 int imparo_load_code_attention_mfma() {
     hipFuncAttributes attributes;
-    return hipFuncGetAttributes(&attributes, reinterpret_cast<const void*>(&k_attn_decode_merge)) == hipSuccess ? IMPARO_OK
+    return hipFuncGetAttributes(&attributes, reinterpret_cast<const void*>(&k_attn_decode_merge<false>)) == hipSuccess ? IMPARO_OK
                                                                                               : IMPARO_LAUNCH_FAILED;
 }

@@ -1,6 +1,7 @@
 // Recurrences with a matrix of state a head and one decay a head and token:
 //   S <- a S + k v^T,                 o = S^T q                  (a linear attention with decay)
 //   S <- a S;  u = b (v - S^T k);  S <- S + k u^T,  o = S^T q    (the gated delta rule)
+//   the same with S <- diag(g) S, one decay a state row          (the gated delta rule, decays a channel)
 // S [dim, vdim] float32 per request and head, carried from token to token. The decay a is a constant of
 // the head, or exp(-rate_h softplus(raw + bias_h)) of a projected number (the step; the values may be
 // multiplied by that step, as a state-space layer does, and the head's result may take D_h x on top). b is
@@ -31,6 +32,8 @@ __device__ __forceinline__ float ds_sigmoid(float z) { return 1.0f / (1.0f + exp
 __device__ __forceinline__ float ds_silu(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float ds_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
+__device__ __forceinline__ float ds_gate(float z, int act) { return act ? ds_sigmoid(z) : ds_silu(z); }
+
 struct DecayScanArgs {
     const float* q; int q_ld, q_off, q_div;      // head h reads q head h / q_div
     const float* k; int k_ld, k_off, k_div;
@@ -49,16 +52,19 @@ struct DecayScanArgs {
     int chunk_tokens, max_chunks;
     float* chunk_state;                          // [rows * max_chunks, heads, dim, vdim]
     float* chunk_decay;                          // [rows * max_chunks, heads]
+    int silu_in;                                 // q, k, v go through SiLU when they are read (token by token only)
 };
 
 // MODE 0: a segment from its request's state to its end. With chunks (blockIdx.x = row * max_chunks + chunk):
 // MODE 1: a chunk that is not the segment's last, from a zero state: its end state goes to chunk_state, the
 // product of its decays to chunk_decay, no results; MODE 2: a chunk from the state chunk_state holds for it,
 // with results; the last chunk writes the request's state.
-// V4: a thread's slice is whole 16-byte pieces, read as such.
-template <int KS, int MODE, bool DELTA, bool V4>
+// V4: a thread's slice is whole 16-byte pieces, read as such. CHAN: step and step_bias hold heads x dim numbers, a
+// decay for every state row.
+template <int KS, int MODE, bool DELTA, bool V4, bool CHAN = false>
 __global__ __launch_bounds__(DS_MAX_THREADS) void k_decay_scan(const DecayScanArgs A) {
     __shared__ __attribute__((aligned(16))) float sq[DS_TOKENS][DS_MAX_DIM], sk[DS_TOKENS][DS_MAX_DIM];
+    __shared__ __attribute__((aligned(16))) float sg[CHAN ? DS_TOKENS : 1][CHAN ? DS_MAX_DIM : 4];
     __shared__ float sv[DS_TOKENS][DS_MAX_THREADS];
     __shared__ float sa[DS_TOKENS], sb[DS_TOKENS], sdt[DS_TOKENS];
     const int VB = blockDim.x / KS;                      // value columns of a block
@@ -96,17 +102,29 @@ __global__ __launch_bounds__(DS_MAX_THREADS) void k_decay_scan(const DecayScanAr
         for (int i = tid; i < nt * dkp; i += blockDim.x) {
             const int tok = i / dkp, k = i - tok * dkp;
             const size_t t = (size_t)(first + t0 + tok);
-            sq[tok][k] = k < dim ? A.q[t * A.q_ld + A.q_off + qh * dim + k] : 0.f;   // beyond dim: a state that stays zero
-            sk[tok][k] = k < dim ? A.k[t * A.k_ld + A.k_off + kh * dim + k] : 0.f;
+            float qv = k < dim ? A.q[t * A.q_ld + A.q_off + qh * dim + k] : 0.f;     // beyond dim: a state that stays zero
+            float kv = k < dim ? A.k[t * A.k_ld + A.k_off + kh * dim + k] : 0.f;
+            if (!DELTA && A.silu_in) qv = ds_silu(qv), kv = ds_silu(kv);
+            sq[tok][k] = qv;
+            sk[tok][k] = kv;
+            if constexpr (CHAN) {
+                const int kc = min(k, dim - 1);
+                sg[tok][k] = expf(-A.rate[h] * ds_softplus(A.step[t * A.step_ld + A.step_off + h * dim + kc] +
+                                                           A.step_bias[h * dim + kc]));
+            }
         }
         for (int i = tid; i < nt * VB; i += blockDim.x) {
             const int tok = i / VB, c = i - tok * VB;
-            sv[tok][c] = (v0 + c) < vdim ? A.v[(size_t)(first + t0 + tok) * A.v_ld + A.v_off + h * vdim + v0 + c] : 0.f;
+            float vv = (v0 + c) < vdim ? A.v[(size_t)(first + t0 + tok) * A.v_ld + A.v_off + h * vdim + v0 + c] : 0.f;
+            if (!DELTA && A.silu_in) vv = ds_silu(vv);
+            sv[tok][c] = vv;
         }
         if (tid < nt) {
             const size_t t = (size_t)(first + t0 + tid);
             float a, dt = 1.f;
-            if (A.decay_const) {
+            if constexpr (CHAN) {
+                a = 1.f;
+            } else if (A.decay_const) {
                 a = A.decay_const[h];
             } else {
                 dt = ds_softplus(A.step[t * A.step_ld + A.step_off + h] + A.step_bias[h]);
@@ -142,10 +160,23 @@ __global__ __launch_bounds__(DS_MAX_THREADS) void k_decay_scan(const DecayScanAr
             }
             if constexpr (DELTA) {
                 float seen = 0.f;
+                float gg[CHAN ? DS_KPT : 1];
+                if constexpr (CHAN) {
+#pragma unroll
+                    for (int j = 0; j < DS_KPT; j += V4 ? 4 : 1)
+                        if (j < kpt) {
+                            if constexpr (V4) {
+                                const float4 g4 = *reinterpret_cast<const float4*>(&sg[tok][ks * kpt + j]);
+                                gg[j] = g4.x, gg[j + 1] = g4.y, gg[j + 2] = g4.z, gg[j + 3] = g4.w;
+                            } else {
+                                gg[j] = sg[tok][ks * kpt + j];
+                            }
+                        }
+                }
 #pragma unroll
                 for (int j = 0; j < DS_KPT; ++j)
                     if (j < kpt) {
-                        S[j] *= a;
+                        S[j] *= CHAN ? gg[CHAN ? j : 0] : a;
                         seen = fmaf(S[j], kk[j], seen);
                     }
 #pragma unroll
@@ -224,6 +255,11 @@ __global__ void k_decay_carry(float* __restrict__ chunk_state, const float* __re
 #define DMAXK 128             // state rows a head at most, in this form
 
 // PLAIN: the recurrence without the delta rule's correction (b = 1, no triangle): M, log g and the steps only.
+// With a decay a state row (CHANNEL) the ratios are numbers of a state row too and stand inside the dot products:
+//   L_tj = b_t sum_i k_ti k_ji g_ti / g_ji,  M_tj = sum_i q_ti k_ji g_ti / g_ji,
+// every ratio the exponential of a difference of logarithms, at most one, so that no decay, however strong, leaves
+// float32's range. The first launch then leaves what the walk multiplies, g_t k_t, g_t q_t, (g_last / g_t) k_t and
+// g_last, beside T and M: T and M [DC, DC], the three [DC, dim4], g_last [dim4], one after the other.
 template <bool PLAIN>
 __global__ __launch_bounds__(256) void k_delta_chunk_prepare(const DecayScanArgs A) {
     __shared__ float sk[DC][DMAXK + 1], sq[DC][DMAXK + 1], sL[PLAIN ? 1 : DC][DC + 1], lg[DC], sb[DC];
@@ -478,6 +514,296 @@ __global__ __launch_bounds__(256) void k_delta_chunk_scan(const DecayScanArgs A)
     }
 }
 
+__host__ __device__ static inline size_t channel_chunk_floats(int dim4) { return 2 * DC * DC + (3 * DC + 1) * (size_t)dim4; }
+
+__global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanArgs A) {
+    __shared__ float sk[DC][DMAXK + 1], sq[DC][DMAXK + 1], lg[DC][DMAXK + 1], sL[DC][DC + 1], sb[DC];
+    const int r = blockIdx.x / A.max_chunks, chunk = blockIdx.x - r * A.max_chunks, h = blockIdx.y;
+    const int tid = threadIdx.x, dim = A.dim, heads = A.heads, dim4 = (dim + 3) & ~3;
+    const int n_all = A.seg_len[r];
+    if (chunk * DC >= n_all) return;                     // (the whole block)
+    const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
+    const int qh = h / A.q_div, kh = h / A.k_div;
+    const float rate = A.rate[h];
+    for (int i = tid; i < DC * dim4; i += 256) {
+        const int t = i / dim4, k = i - t * dim4;
+        const bool on = t < n && k < dim;
+        const size_t row = (size_t)(first + min(t, n - 1));
+        const int kc = min(k, dim - 1);
+        const float kv = A.k[row * A.k_ld + A.k_off + kh * dim + kc], qv = A.q[row * A.q_ld + A.q_off + qh * dim + kc];
+        const float raw = A.step[row * A.step_ld + A.step_off + h * dim + kc] + A.step_bias[h * dim + kc];
+        sk[t][k] = on ? kv : 0.f;
+        sq[t][k] = on ? qv : 0.f;
+        lg[t][k] = on ? -rate * ds_softplus(raw) : 0.f;
+    }
+    if (tid < DC)
+        sb[tid] = tid < n ? ds_sigmoid(A.beta[(size_t)(first + tid) * A.beta_ld + A.beta_off + h]) : 0.f;
+    __syncthreads();
+    if (tid < dim4) {
+        float sum = 0.f;
+        for (int t = 0; t < DC; ++t) {
+            sum += lg[t][tid];
+            lg[t][tid] = sum;
+        }
+    }
+    __syncthreads();
+    float* T_out = A.chunk_state + ((size_t)blockIdx.x * heads + h) * channel_chunk_floats(dim4);
+    float* M_out = T_out + DC * DC;
+    float* kg_out = M_out + DC * DC;
+    float* qg_out = kg_out + DC * dim4;
+    float* ke_out = qg_out + DC * dim4;
+    for (int i = tid; i < DC * DC; i += 256) {
+        const int t = i / DC, j = i - t * DC;
+        float kk = 0.f, qk = 0.f;
+        if (j <= t) {
+#pragma unroll 4
+            for (int k = 0; k < dim; ++k) {
+                const float w = sk[j][k] * expf(lg[t][k] - lg[j][k]);
+                kk = fmaf(sk[t][k], w, kk);
+                qk = fmaf(sq[t][k], w, qk);
+            }
+        }
+        sL[t][j] = j < t ? kk * sb[t] : 0.f;
+        M_out[i] = qk;
+    }
+    for (int i = tid; i < DC * dim4; i += 256) {
+        const int t = i / dim4, k = i - t * dim4;
+        const float g = expf(lg[t][k]);
+        kg_out[i] = sk[t][k] * g;
+        qg_out[i] = sq[t][k] * g;
+        ke_out[i] = sk[t][k] * expf(lg[DC - 1][k] - lg[t][k]);
+    }
+    if (tid < dim4) ke_out[DC * dim4 + tid] = expf(lg[DC - 1][tid]);
+    __syncthreads();
+    if (tid < DC) {
+        // column tid of (I + L)^-1 by forward substitution, then times b of that column
+        float x[DC];
+#pragma unroll
+        for (int t = 0; t < DC; ++t) {
+            float acc = t == tid ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < t; ++j) acc = fmaf(-sL[t][j], x[j], acc);
+            x[t] = acc;
+        }
+        const float b = sb[tid];
+#pragma unroll
+        for (int t = 0; t < DC; ++t) T_out[t * DC + tid] = x[t] * b;
+    }
+}
+
+// The walk: a segment's chunks in order with the state in LDS, a block a (segment, head, run of VB value columns).
+template <int VB>
+__global__ __launch_bounds__(256) void k_channel_delta_scan(const DecayScanArgs A) {
+    constexpr int KLD = DMAXK + 4;                       // floats between two tokens' rows: whole 16-byte pieces
+    constexpr int NG = 256 / VB;                         // threads a value column: each takes every NG-th token
+    constexpr int TPT = DC / NG;                         // tokens of a chunk a thread takes
+    constexpr int KPT = DMAXK / NG;                      // state rows of its column a thread takes at most
+    constexpr int PIECES = DC * DMAXK / 4 / 256;         // 16-byte pieces of a chunk's rows a thread brings at most
+    __shared__ __attribute__((aligned(16))) float sk[DC][KLD], sq[DC][KLD];
+    __shared__ __attribute__((aligned(16))) float sT[DC][DC], sM[DC][DC];
+    __shared__ float sS[DMAXK][VB], sU[DC][VB], gl[DMAXK];
+    float (*sR)[VB] = reinterpret_cast<float (*)[VB]>(&sq[0][0]);        // R lies where Q lay, once Q has been used
+    const int r = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VB;
+    const int tid = threadIdx.x, v = tid % VB, g = tid / VB;
+    const int heads = A.heads, dim = A.dim, vdim = A.vdim;
+    const int dim4 = (dim + 3) & ~3, pieces = DC * dim4 / 4;
+    const bool live = v0 + v < vdim;
+    const int n_all = A.seg_len[r], n_chunks = (n_all + DC - 1) / DC;
+    const size_t floats = channel_chunk_floats(dim4);
+    float* S_at = A.state + (((size_t)A.slot[r] * heads + h) * dim) * vdim;
+    for (int i = tid; i < dim4 * VB; i += 256) {
+        const int k = i / VB, c = i - k * VB;
+        sS[k][c] = (k < dim && (v0 + c) < vdim) ? S_at[(size_t)k * vdim + v0 + c] : 0.f;
+    }
+    float4 fk[PIECES], fq[PIECES], fe[PIECES], ft, fm;
+    float fv[TPT], fl;
+    // every address is clamped (no load under a branch)
+    auto fetch = [&](int chunk) {
+        const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
+        const float* at = A.chunk_state + ((size_t)(r * A.max_chunks + chunk) * heads + h) * floats;
+        ft = *reinterpret_cast<const float4*>(at + 4 * tid);
+        fm = *reinterpret_cast<const float4*>(at + DC * DC + 4 * tid);
+        const float* kg = at + 2 * DC * DC;
+#pragma unroll
+        for (int it = 0; it < PIECES; ++it) {
+            const int p = min(tid + 256 * it, pieces - 1);
+            fk[it] = *reinterpret_cast<const float4*>(kg + 4 * p);
+            fq[it] = *reinterpret_cast<const float4*>(kg + DC * dim4 + 4 * p);
+            fe[it] = *reinterpret_cast<const float4*>(kg + 2 * DC * dim4 + 4 * p);
+        }
+        fl = kg[3 * DC * dim4 + min(tid, dim4 - 1)];
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) {
+            const int t = min(g + NG * i, n - 1);
+            fv[i] = A.v[(size_t)(first + t) * A.v_ld + A.v_off + h * vdim + min(v0 + v, vdim - 1)];
+        }
+    };
+    fetch(0);
+    const int kpt = (((dim4 + NG - 1) / NG) + 3) & ~3;   // this thread's state rows: kpt from g * kpt on
+    for (int chunk = 0; chunk < n_chunks; ++chunk) {
+        const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
+        __syncthreads();                                 // the chunk before has been used, the state is whole
+        float4 ke[PIECES];
+#pragma unroll
+        for (int it = 0; it < PIECES; ++it) {
+            const int p = tid + 256 * it, t = p / (dim4 / 4), k = (p - t * (dim4 / 4)) * 4;
+            if (p < pieces) {
+                *reinterpret_cast<float4*>(&sk[t][k]) = fk[it];
+                *reinterpret_cast<float4*>(&sq[t][k]) = fq[it];
+            }
+            ke[it] = fe[it];
+        }
+        *reinterpret_cast<float4*>(&sT[tid / (DC / 4)][tid % (DC / 4) * 4]) = ft;
+        *reinterpret_cast<float4*>(&sM[tid / (DC / 4)][tid % (DC / 4) * 4]) = fm;
+        if (tid < dim4) gl[tid] = fl;
+        float vt[TPT];
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) vt[i] = (g + NG * i < n && live) ? fv[i] : 0.f;
+        __syncthreads();
+        fetch(min(chunk + 1, n_chunks - 1));             // on its way while this chunk is worked on (no load under a branch)
+        // what the decayed state says of the chunk's keys and queries
+        float p[TPT], s[TPT];
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) p[i] = s[i] = 0.f;
+#pragma unroll 4
+        for (int k = 0; k < dim4; k += 4) {
+            const float s0 = sS[k][v], s1 = sS[k + 1][v], s2 = sS[k + 2][v], s3 = sS[k + 3][v];
+#pragma unroll
+            for (int i = 0; i < TPT; ++i) {
+                const float4 kk = *reinterpret_cast<const float4*>(&sk[g + NG * i][k]);
+                const float4 qq = *reinterpret_cast<const float4*>(&sq[g + NG * i][k]);
+                p[i] = fmaf(kk.w, s3, fmaf(kk.z, s2, fmaf(kk.y, s1, fmaf(kk.x, s0, p[i]))));
+                s[i] = fmaf(qq.w, s3, fmaf(qq.z, s2, fmaf(qq.y, s1, fmaf(qq.x, s0, s[i]))));
+            }
+        }
+        __syncthreads();                                 // K and Q have been used: R goes where Q lay, the weighed keys where K lay
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) sR[g + NG * i][v] = vt[i] - p[i];
+#pragma unroll
+        for (int it = 0; it < PIECES; ++it) {
+            const int pc = tid + 256 * it, t = pc / (dim4 / 4), k = (pc - t * (dim4 / 4)) * 4;
+            if (pc < pieces) *reinterpret_cast<float4*>(&sk[t][k]) = ke[it];
+        }
+        __syncthreads();
+        // (T and M are zero above their diagonals: the sums run over the whole chunk, so that the reads of
+        // several steps can be under way at once; a product with zero adds nothing)
+        float u[TPT];
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) u[i] = 0.f;
+#pragma unroll 8
+        for (int j = 0; j < DC; ++j) {
+            const float rv = sR[j][v];
+#pragma unroll
+            for (int i = 0; i < TPT; ++i) u[i] = fmaf(sT[g + NG * i][j], rv, u[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) sU[g + NG * i][v] = u[i];
+        __syncthreads();
+#pragma unroll 8
+        for (int j = 0; j < DC; ++j) {
+            const float uv = sU[j][v];
+#pragma unroll
+            for (int i = 0; i < TPT; ++i) s[i] = fmaf(sM[g + NG * i][j], uv, s[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < TPT; ++i) {
+            const int t = g + NG * i;
+            if (t < n && live) A.out[(size_t)(first + t) * heads * vdim + (size_t)h * vdim + v0 + v] = s[i];
+        }
+        // the state behind the chunk: this thread's rows of its column
+        float acc[KPT];
+#pragma unroll
+        for (int m = 0; m < KPT; ++m)
+            acc[m] = (m < kpt && g * kpt + m < dim4) ? gl[g * kpt + m] * sS[g * kpt + m][v] : 0.f;
+#pragma unroll 4
+        for (int j = 0; j < DC; ++j) {
+            const float uv = sU[j][v];
+#pragma unroll
+            for (int m = 0; m < KPT; m += 4)
+                if (m < kpt && g * kpt + m < dim4) {
+                    const float4 w = *reinterpret_cast<const float4*>(&sk[j][g * kpt + m]);
+                    acc[m] = fmaf(w.x, uv, acc[m]);
+                    acc[m + 1] = fmaf(w.y, uv, acc[m + 1]);
+                    acc[m + 2] = fmaf(w.z, uv, acc[m + 2]);
+                    acc[m + 3] = fmaf(w.w, uv, acc[m + 3]);
+                }
+        }
+#pragma unroll
+        for (int m = 0; m < KPT; ++m)
+            if (m < kpt && g * kpt + m < dim4) sS[g * kpt + m][v] = acc[m];
+    }
+    __syncthreads();
+    for (int i = tid; i < dim * VB; i += 256) {
+        const int k = i / VB, c = i - k * VB;
+        if (v0 + c < vdim) S_at[(size_t)k * vdim + v0 + c] = sS[k][c];
+    }
+}
+
+extern "C" long long imparo_channel_delta_scratch(int dim) { return (long long)channel_chunk_floats((dim + 3) & ~3); }
+
+extern "C" int imparo_channel_delta_scan(const float* q, int q_ld, int q_off, int q_div, const float* k, int k_ld,
+                                         int k_off, int k_div, const float* v, int v_ld, int v_off, const float* step,
+                                         int step_ld, int step_off, const float* step_bias, const float* rate,
+                                         const float* beta, int beta_ld, int beta_off, float* state,
+                                         const int32_t* seg_start, const int32_t* seg_len, const int32_t* slot,
+                                         float* out, int n_rows, int heads, int dim, int vdim, int chunk_tokens,
+                                         int max_chunks, float* scratch, imparo_stream stream) {
+    if (!q || !k || !v || !step || !step_bias || !rate || !beta || !state || !seg_start || !seg_len || !slot || !out)
+        return IMPARO_BAD_ARGUMENT;
+    if (chunk_tokens && (chunk_tokens != DC || dim > DMAXK || max_chunks < 1 || !scratch || ((uintptr_t)scratch & 15)))
+        return IMPARO_BAD_ARGUMENT;
+    if (n_rows < 0 || heads < 1 || dim < 1 || dim > DS_MAX_DIM || vdim < 1) return IMPARO_BAD_ARGUMENT;
+    if (q_div < 1 || k_div < 1 || heads % q_div || heads % k_div) return IMPARO_BAD_ARGUMENT;
+    if (q_off < 0 || k_off < 0 || v_off < 0 || q_ld < q_off + heads / q_div * dim || k_ld < k_off + heads / k_div * dim ||
+        v_ld < v_off + heads * vdim || step_off < 0 || step_ld < step_off + heads * dim || beta_off < 0 ||
+        beta_ld < beta_off + heads)
+        return IMPARO_BAD_ARGUMENT;
+    if (n_rows == 0) return IMPARO_OK;
+    if ((long long)n_rows * (chunk_tokens ? max_chunks : 1) > 0x7fffffffLL) return IMPARO_BAD_ARGUMENT;
+    hipStream_t s = (hipStream_t)stream;
+    int ks = 1;
+    while ((dim + ks - 1) / ks > DS_KPT) ks *= 2;
+    const int kpt = (dim + ks - 1) / ks;
+    DecayScanArgs args{};
+    args.q = q, args.q_ld = q_ld, args.q_off = q_off, args.q_div = q_div;
+    args.k = k, args.k_ld = k_ld, args.k_off = k_off, args.k_div = k_div;
+    args.v = v, args.v_ld = v_ld, args.v_off = v_off;
+    args.step = step, args.step_ld = step_ld, args.step_off = step_off, args.step_bias = step_bias, args.rate = rate;
+    args.beta = beta, args.beta_ld = beta_ld, args.beta_off = beta_off;
+    args.state = state, args.seg_start = seg_start, args.seg_len = seg_len, args.slot = slot, args.out = out;
+    args.heads = heads, args.dim = dim, args.vdim = vdim, args.kpt = kpt;
+    args.chunk_tokens = chunk_tokens, args.max_chunks = max_chunks, args.chunk_state = scratch;
+    if (chunk_tokens) {
+        k_channel_delta_prepare<<<dim3(n_rows * max_chunks, heads), 256, 0, s>>>(args);
+        // few blocks (a segment, few heads): narrower runs of columns make more of them
+        const long long rh = (long long)n_rows * heads;
+#define CDS(VB) k_channel_delta_scan<VB><<<dim3(n_rows, heads, (vdim + VB - 1) / VB), 256, 0, s>>>(args)
+        if (rh * ((vdim + 31) / 32) >= 512) CDS(32);
+        else if (rh * ((vdim + 15) / 16) >= 512) CDS(16);
+        else CDS(8);
+#undef CDS
+        return launch_status();
+    }
+    int threads = (ks * vdim + WAVE - 1) / WAVE * WAVE;
+    threads = threads > DS_MAX_THREADS ? DS_MAX_THREADS : threads;
+    const int vb = threads / ks;
+    const dim3 grid(n_rows, heads, (vdim + vb - 1) / vb);
+#define CDS_WALK(KS)                                                                                                 \
+    if (kpt % 4 == 0) k_decay_scan<KS, 0, true, true, true><<<grid, threads, 0, s>>>(args);                         \
+    else k_decay_scan<KS, 0, true, false, true><<<grid, threads, 0, s>>>(args)
+    switch (ks) {
+        case 1: CDS_WALK(1); break;
+        case 2: CDS_WALK(2); break;
+        case 4: CDS_WALK(4); break;
+        case 8: CDS_WALK(8); break;
+        case 16: CDS_WALK(16); break;
+        case 32: CDS_WALK(32); break;
+        default: return IMPARO_BAD_ARGUMENT;
+    }
+#undef CDS_WALK
+    return launch_status();
+}
+
 extern "C" int imparo_delta_chunk_tokens() { return DC; }
 extern "C" int imparo_delta_chunk_max_dim() { return DMAXK; }
 
@@ -487,8 +813,9 @@ extern "C" int imparo_decay_scan(const float* q, int q_ld, int q_off, int q_div,
                                  const float* rate, int v_times_step, const float* beta, int beta_ld, int beta_off,
                                  const float* skip, float* state, const int32_t* seg_start, const int32_t* seg_len,
                                  const int32_t* slot, float* out, int n_rows, int heads, int dim, int vdim,
-                                 int chunk_tokens, int max_chunks, float* chunk_state, float* chunk_decay,
+                                 int chunk_tokens, int max_chunks, float* chunk_state, float* chunk_decay, int silu_in,
                                  imparo_stream stream) {
+    if (silu_in && (chunk_tokens || beta)) return IMPARO_BAD_ARGUMENT;
     if (!q || !k || !v || !state || !seg_start || !seg_len || !slot || !out) return IMPARO_BAD_ARGUMENT;
     if (!decay_const && (!step || !step_bias || !rate)) return IMPARO_BAD_ARGUMENT;
     if (v_times_step && decay_const) return IMPARO_BAD_ARGUMENT;
@@ -518,7 +845,7 @@ extern "C" int imparo_decay_scan(const float* q, int q_ld, int q_off, int q_div,
     const DecayScanArgs args{q, q_ld, q_off, q_div, k, k_ld, k_off, k_div, v, v_ld, v_off, decay_const,
                              step, step_ld, step_off, step_bias, rate, v_times_step, beta, beta_ld, beta_off, skip,
                              state, seg_start, seg_len, slot, out, heads, dim, vdim, kpt,
-                             chunk_tokens, max_chunks, chunk_state, chunk_decay};
+                             chunk_tokens, max_chunks, chunk_state, chunk_decay, silu_in};
     if (chunk_tokens == DC && dim <= DMAXK) {
         // the chunks of a segment in order, small products a chunk: chunk_state holds T and M of every chunk,
         // chunk_decay the logarithms of its decays and its steps
@@ -570,6 +897,34 @@ extern "C" int imparo_decay_scan(const float* q, int q_ld, int q_off, int q_div,
     return launch_status();
 }
 
+// ---------------------------------------------------------------- columns before the walk
+// SiLU in place on n columns from off on of float32 rows; V neighbouring columns a thread.
+template <int V>
+__global__ void k_silu_columns(float* __restrict__ rows, int ld, int off, int n, long long total) {
+    const int per_row = n / V;
+    const long long id = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (id >= total) return;
+    const long long t = id / per_row;
+    float* p = rows + t * ld + off + (id - t * per_row) * V;
+    if constexpr (V == 4) {
+        float4 x = *reinterpret_cast<const float4*>(p);
+        *reinterpret_cast<float4*>(p) = make_float4(ds_silu(x.x), ds_silu(x.y), ds_silu(x.z), ds_silu(x.w));
+    } else {
+        *p = ds_silu(*p);
+    }
+}
+
+extern "C" int imparo_silu_columns(float* rows, int ld, int off, int n, int n_tokens, imparo_stream stream) {
+    if (!rows || off < 0 || n < 1 || ld < off + n || n_tokens < 0) return IMPARO_BAD_ARGUMENT;
+    if (n_tokens == 0) return IMPARO_OK;
+    const bool four = n % 4 == 0 && off % 4 == 0 && ld % 4 == 0 && !((uintptr_t)rows & 15);
+    const long long total = (long long)n_tokens * (four ? n / 4 : n);
+    const unsigned blocks = (unsigned)((total + 255) / 256);
+    if (four) k_silu_columns<4><<<blocks, 256, 0, (hipStream_t)stream>>>(rows, ld, off, n, total);
+    else k_silu_columns<1><<<blocks, 256, 0, (hipStream_t)stream>>>(rows, ld, off, n, total);
+    return launch_status();
+}
+
 // ---------------------------------------------------------------- a head before the walk
 // One wave per (token, head) over rows [tokens, ld] float32, in place: head j is the `dim` columns from
 // off + j dim. `unit`: the head is divided by sqrt(sum of its squares + unit_eps). Then the first 2 n_freq
@@ -617,7 +972,8 @@ extern "C" int imparo_head_prepare(float* rows, int ld, int off, int n_tokens, i
 }
 
 // ---------------------------------------------------------------- the heads behind the walk
-// out[t, c] for a row of `width` values in `groups` equal parts: with y = x[t, c] and g = silu(gate[t, c]),
+// out[t, c] for a row of `width` values in `groups` equal parts: with y = x[t, c] and g = silu(gate[t, c]) (gate_act
+// 1: its sigmoid),
 //   gate_first: (y g) / rms_part(y g) * w[c];   otherwise: y / rms_part(y) * w[c] * g     (w null: 1).
 // A wave takes a part; for long parts a block does, with the part in registers (PER values a thread, every load
 // asked for before any is used, the gate's activation taken once).
@@ -625,7 +981,7 @@ template <typename TOut>
 __global__ __launch_bounds__(256) void k_gated_group_norm(const float* __restrict__ x, const float* __restrict__ gate,
                                                           int gate_ld, int gate_off, const float* __restrict__ w,
                                                           TOut* __restrict__ out, int n_tokens, int width, int groups,
-                                                          float eps, int gate_first) {
+                                                          float eps, int gate_first, int gate_act) {
     const int part = width / groups;
     const long long id = (long long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
     const int first = threadIdx.x & (WAVE - 1);
@@ -637,7 +993,7 @@ __global__ __launch_bounds__(256) void k_gated_group_norm(const float* __restric
 #pragma unroll 4
     for (int i = first; i < part; i += WAVE) {
         float y = xr[i];
-        if (gate_first && gr) y *= ds_silu(gr[i]);
+        if (gate_first && gr) y *= ds_gate(gr[i], gate_act);
         ss = fmaf(y, y, ss);
     }
     ss = wave_sum(ss);
@@ -645,7 +1001,7 @@ __global__ __launch_bounds__(256) void k_gated_group_norm(const float* __restric
 #pragma unroll 4
     for (int i = first; i < part; i += WAVE) {
         float y = xr[i];
-        const float gv = gr ? ds_silu(gr[i]) : 1.f;
+        const float gv = gr ? ds_gate(gr[i], gate_act) : 1.f;
         if (gate_first) y *= gv;
         y = y * rs * (w ? w[(size_t)g * part + i] : 1.f);
         if (!gate_first) y *= gv;
@@ -657,7 +1013,7 @@ template <typename TOut, int PER>
 __global__ __launch_bounds__(256) void k_gated_group_norm_block(const float* __restrict__ x, const float* __restrict__ gate,
                                                                 int gate_ld, int gate_off, const float* __restrict__ w,
                                                                 TOut* __restrict__ out, int width, int groups, float eps,
-                                                                int gate_first) {
+                                                                int gate_first, int gate_act) {
     __shared__ float scratch[16];
     const int part = width / groups;
     const int t = blockIdx.x / groups, g = blockIdx.x - t * groups;
@@ -674,7 +1030,7 @@ __global__ __launch_bounds__(256) void k_gated_group_norm_block(const float* __r
     float ss = 0.f;
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
-        gv[j] = gr ? ds_silu(gv[j]) : 1.f;
+        gv[j] = gr ? ds_gate(gv[j], gate_act) : 1.f;
         if (gate_first) y[j] *= gv[j];
         if ((int)threadIdx.x + j * 256 < part) ss = fmaf(y[j], y[j], ss);
     }
@@ -690,7 +1046,8 @@ __global__ __launch_bounds__(256) void k_gated_group_norm_block(const float* __r
 
 extern "C" int imparo_gated_group_norm(const float* x, const float* gate, int gate_ld, int gate_off, const float* w,
                                        void* out, int out_dtype, int n_tokens, int width, int groups, float eps,
-                                       int gate_first, imparo_stream stream) {
+                                       int gate_first, int gate_act, imparo_stream stream) {
+    if (gate_act != 0 && gate_act != 1) return IMPARO_BAD_ARGUMENT;
     if (!x || !out || n_tokens < 0 || width < 1 || groups < 1 || width % groups) return IMPARO_BAD_ARGUMENT;
     if (gate && (gate_off < 0 || gate_ld < gate_off + width)) return IMPARO_BAD_ARGUMENT;
     if (out_dtype != IMPARO_F32 && out_dtype != IMPARO_BF16) return IMPARO_BAD_ARGUMENT;
@@ -702,7 +1059,7 @@ extern "C" int imparo_gated_group_norm(const float* x, const float* gate, int ga
     if (part > 512 && part <= 256 * 64) {
 #define GGN_BLOCK(T, PER)                                                                                            \
     k_gated_group_norm_block<T, PER><<<(unsigned)parts, 256, 0, s>>>(x, gate, gate_ld, gate_off, w, (T*)out, width, \
-                                                                     groups, eps, gate_first)
+                                                                     groups, eps, gate_first, gate_act)
 #define GGN_PER(T)                                                                                                   \
     if (part <= 256 * 4) GGN_BLOCK(T, 4);                                                                            \
     else if (part <= 256 * 8) GGN_BLOCK(T, 8);                                                                       \
@@ -717,10 +1074,10 @@ extern "C" int imparo_gated_group_norm(const float* x, const float* gate, int ga
     const unsigned blocks = (unsigned)((parts + 3) / 4);
     if (out_dtype == IMPARO_BF16)
         k_gated_group_norm<bf16_t><<<blocks, 256, 0, s>>>(x, gate, gate_ld, gate_off, w, (bf16_t*)out, n_tokens, width,
-                                                          groups, eps, gate_first);
+                                                          groups, eps, gate_first, gate_act);
     else
         k_gated_group_norm<float><<<blocks, 256, 0, s>>>(x, gate, gate_ld, gate_off, w, (float*)out, n_tokens, width,
-                                                         groups, eps, gate_first);
+                                                         groups, eps, gate_first, gate_act);
     return launch_status();
 }
 

@@ -25,6 +25,16 @@ union Frag8 {
 #define EPI_SWIGLU 1   // weight rows interleaved gate, up, gate, up...: out[m, j] = silu(y[m, 2j]) * y[m, 2j+1]
 #define EPI_ADD 2      // float32 out only: Y += y, what Y holds being read where the result is stored
 
+// What happens to a product before it is stored: its kind (one of the above) and, for the SwiGLU kind, a constant
+// the result is multiplied by in float32 before it is rounded (a factor on the whole sublayer, carried by the input
+// of the product that follows).
+struct Epilogue {
+    int kind;
+    float scale;
+    __host__ __device__ Epilogue(int k, float s = 1.0f) : kind(k), scale(s) {}
+    __host__ __device__ operator int() const { return kind; }
+};
+
 __device__ __forceinline__ float silu_mul_f(float g, float u) { return g / (1.0f + expf(-g)) * u; }
 // The same with the hardware's exp2 and reciprocal (an ulp each) for the bfloat16 kernels: the exact
 // division and exponential cost some thirty instructions per output, ten microseconds per 256x256 tile
@@ -44,7 +54,7 @@ __device__ __forceinline__ uint4 zero_if(bool out, uint4 v) {
 template <typename TOut>
 __global__ __launch_bounds__(256) void k_gemm_f32(const float* __restrict__ X, const float* __restrict__ W,
                                                   const float* __restrict__ bias, TOut* __restrict__ Y,
-                                                  int M, int N, int K, int epilogue) {
+                                                  int M, int N, int K, Epilogue epilogue) {
     __shared__ float As[F32_BK][F32_BM + 4];
     __shared__ float Bs[F32_BK][F32_BN + 4];
     const int tid = threadIdx.x;
@@ -97,7 +107,7 @@ __global__ __launch_bounds__(256) void k_gemm_f32(const float* __restrict__ X, c
 #pragma unroll
             for (int j = 0; j < 4; j += 2) {
                 const int n = n0 + tx * 4 + j;
-                if (n + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_f(acc[i][j], acc[i][j + 1]));
+                if (n + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_f(acc[i][j], acc[i][j + 1]) * epilogue.scale);
             }
             continue;
         }
@@ -119,7 +129,7 @@ __global__ __launch_bounds__(256) void k_gemm_f32(const float* __restrict__ X, c
 template <typename TOut>
 __global__ __launch_bounds__(256) void k_gemm_f32_rows(const float* __restrict__ X, const float* __restrict__ W,
                                                        const float* __restrict__ bias, TOut* __restrict__ Y,
-                                                       int M, int N, int K, int epilogue) {
+                                                       int M, int N, int K, Epilogue epilogue) {
     __shared__ float Ws[F32R_BK][F32R_BN + 1];
     __shared__ float Xs[F32R_BK][16 + 1];
     const int tid = threadIdx.x;
@@ -170,7 +180,7 @@ __global__ __launch_bounds__(256) void k_gemm_f32_rows(const float* __restrict__
         if (n + 1 < N) acc1 += bias[n + 1];
     }
     if (epilogue == EPI_SWIGLU) {
-        if (n + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_f(acc0, acc1));
+        if (n + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_f(acc0, acc1) * epilogue.scale);
         return;
     }
     if (n < N) store_f32<TOut>(Y, (size_t)m * N + n, acc0);
@@ -195,7 +205,7 @@ template <typename TOut>
 __global__ __launch_bounds__(256, 2) void k_gemm_bf16_tile(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
                                                            const float* __restrict__ bias, TOut* __restrict__ Y,
                                                            int M, int N, int K_all, int tiles_m, int tiles_n,
-                                                           int epilogue, int k_per) {
+                                                           Epilogue epilogue, int k_per) {
     __shared__ __attribute__((aligned(16))) bf16_t As[2][BG_BM * BG_LD];
     __shared__ __attribute__((aligned(16))) bf16_t Bs[2][BG_BN * BG_LD];
     // slices of K (gridDim.y > 1): block (x, y) sums K range [y * k_per, (y+1) * k_per) into Y + y * M * N
@@ -348,7 +358,7 @@ __global__ __launch_bounds__(256, 2) void k_gemm_bf16_tile(const bf16_t* __restr
                     const float other = __shfl_xor(mine, 1, WAVE);
                     const int m = m0 + wm * 64 + i * 32 + (r >> 2) * 8 + (lane >> 5) * 4 + (r & 3);
                     if (!(lane & 1) && n + 1 < N && m < M)
-                        store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_fast(mine, other));
+                        store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_fast(mine, other) * epilogue.scale);
                 }
                 continue;
             }
@@ -377,7 +387,7 @@ __global__ __launch_bounds__(WM * WN * 64) void k_gemm_bf16_big(const bf16_t* __
                                                                 const bf16_t* __restrict__ W,
                                                                 const float* __restrict__ bias,
                                                                 TOut* __restrict__ Y, int M, int N, int K,
-                                                                int tiles_m, int tiles_n, int epilogue) {
+                                                                int tiles_m, int tiles_n, Epilogue epilogue) {
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32, NT = WM * WN * 64;
     constexpr int PA = BM * 8 / NT, PB = BN * 8 / NT;      // 16-byte pieces of a K-step per thread
     static_assert(BM * 8 % NT == 0 && BN * 8 % NT == 0, "tile rows must divide over the threads");
@@ -495,7 +505,7 @@ __global__ __launch_bounds__(WM * WN * 64) void k_gemm_bf16_big(const bf16_t* __
                     const float other = __shfl_xor(mine, 1, WAVE);
                     const int m = m0 + (wm * TM + i) * 32 + (r >> 2) * 8 + (lane >> 5) * 4 + (r & 3);
                     if (!(lane & 1) && n + 1 < N && m < M)
-                        store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_fast(mine, other));
+                        store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_fast(mine, other) * epilogue.scale);
                 }
                 continue;
             }
@@ -509,7 +519,7 @@ __global__ __launch_bounds__(WM * WN * 64) void k_gemm_bf16_big(const bf16_t* __
 }
 
 template <typename TOut, int WM, int WN, int TM, int TN>
-static int launch_big(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k, int epilogue,
+static int launch_big(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k, Epilogue epilogue,
                       hipStream_t s) {
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32;
     constexpr size_t lds_bytes = (size_t)2 * (BM + BN) * BG_LD * sizeof(bf16_t);
@@ -597,7 +607,7 @@ template <typename TOut, int TMI, int TN, int NWN, int NWM = 2, int STAGES = 2>
 __global__ __launch_bounds__(64 * NWM * NWN) void k_gemm_bf16_dma(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W,
                                                              const float* __restrict__ bias, TOut* __restrict__ Y,
                                                              int M, int N, int K_all, int k_per, int tiles_m,
-                                                             int tiles_n, int epilogue) {
+                                                             int tiles_n, Epilogue epilogue) {
     constexpr int NW = NWM * NWN;                      // waves of the block
     constexpr int WN = 32 * TN;                        // weight rows of one wave's part
     constexpr int BN = NWN * WN;                       // of the block's tile
@@ -804,8 +814,8 @@ __global__ __launch_bounds__(64 * NWM * NWN) void k_gemm_bf16_dma(const bf16_t* 
             const int m = m0 + wm * WM + i * 32 + row;
             float o[4] = {v.x + bn[0], v.y + bn[1], v.z + bn[2], v.w + bn[3]};
             if (swiglu) {
-                o[0] = silu_mul_fast(o[0], o[1]);
-                o[1] = silu_mul_fast(o[2], o[3]);
+                o[0] = silu_mul_fast(o[0], o[1]) * epilogue.scale;
+                o[1] = silu_mul_fast(o[2], o[3]) * epilogue.scale;
             }
             TOut* dst = Y + (size_t)m * out_n + (swiglu ? n / 2 : n);
             if (vectors) {
@@ -915,7 +925,7 @@ static DmaPlan dma_plan(int m, int n, int k, int fixed_slices) {
 // `slices` must leave every slice a multiple of 128 of K (dma_tile_takes(m, n, k / slices) and k % slices == 0).
 // bm: 256 or 128 activation rows to a tile; tn: 4, 3 (bm 256 only), 2 or 1 (bm 128 only) for 256, 192, 128 or 64 weight rows.
 template <typename TOut>
-static int launch_dma(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k, int epilogue,
+static int launch_dma(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k, Epilogue epilogue,
                       int bm, int tn, int slices, hipStream_t s, int stages = 2) {
     const int tiles_m = (m + bm - 1) / bm, tiles_n = (n + 64 * tn - 1) / (64 * tn);
     const long long total = (long long)tiles_m * tiles_n;
@@ -966,7 +976,7 @@ __global__ __launch_bounds__(NW * 64) void k_gemm_bf16_skinny(const bf16_t* __re
                                                               const bf16_t* __restrict__ W,
                                                               const float* __restrict__ bias,
                                                               TOut* __restrict__ Y, int M, int N, int K_all,
-                                                              int k_per, int epilogue) {
+                                                              int k_per, Epilogue epilogue) {
     __shared__ float red[NW][MT][64][4];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int n0 = blockIdx.x * 16;
@@ -1039,7 +1049,7 @@ __global__ __launch_bounds__(NW * 64) void k_gemm_bf16_skinny(const bf16_t* __re
 #pragma unroll
             for (int i = 0; i < 4; i += 2) {
                 const int n = n0 + g * 4 + i;
-                if (n + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_fast(v[i], v[i + 1]));
+                if (n + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + n / 2, silu_mul_fast(v[i], v[i + 1]) * epilogue.scale);
             }
             continue;
         }
@@ -1053,7 +1063,7 @@ __global__ __launch_bounds__(NW * 64) void k_gemm_bf16_skinny(const bf16_t* __re
 
 template <typename TOut, int MT>
 static void launch_skinny(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k,
-                          int epilogue, int slices, hipStream_t s) {
+                          Epilogue epilogue, int slices, hipStream_t s) {
     const int k_per = ((k + slices - 1) / slices + 127) / 128 * 128;
     dim3 grid((unsigned)((n + 15) / 16), (unsigned)((k + k_per - 1) / k_per));
     // few chunks of 128 per wave: 4 waves up to 512 of K per block, 8 up to 2048, 16 beyond
@@ -1354,7 +1364,7 @@ struct StreamSet {
 template <typename TOut, int MT, int ST_WAVES>
 __global__ __launch_bounds__(ST_WAVES * 64) void k_gemm_bf16_stream(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, const float* __restrict__ bias,
-    TOut* __restrict__ Y, int M, int N, int K_all, int k_per, int epilogue, const float* __restrict__ ssq_in,
+    TOut* __restrict__ Y, int M, int N, int K_all, int k_per, Epilogue epilogue, const float* __restrict__ ssq_in,
     int n_parts, float eps) {
     __shared__ __attribute__((aligned(16))) bf16_t xs[2][MT * 16 * ST_LD];
     __shared__ float norm_part[ST_WAVES * 4 * 16];
@@ -1490,7 +1500,7 @@ __global__ __launch_bounds__(ST_WAVES * 64) void k_gemm_bf16_stream(
         if (epilogue == EPI_SWIGLU) {
 #pragma unroll
             for (int i = 0; i < 4; i += 2)
-                if (nq + i + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + (nq + i) / 2, silu_mul_fast(v[i], v[i + 1]));
+                if (nq + i + 1 < N) store_f32<TOut>(Y, (size_t)m * (N / 2) + (nq + i) / 2, silu_mul_fast(v[i], v[i + 1]) * epilogue.scale);
             continue;
         }
 #pragma unroll
@@ -1501,7 +1511,7 @@ __global__ __launch_bounds__(ST_WAVES * 64) void k_gemm_bf16_stream(
 
 template <typename TOut, int MT>
 static void launch_stream(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k,
-                          int epilogue, int nw, int slices, hipStream_t s, const float* ssq_in = nullptr,
+                          Epilogue epilogue, int nw, int slices, hipStream_t s, const float* ssq_in = nullptr,
                           int n_parts = 0, float eps = 0.f) {
     const int k_per = ((k + slices - 1) / slices + ST_BK - 1) / ST_BK * ST_BK;
     dim3 grid((unsigned)((n + nw * 16 - 1) / (nw * 16)), (unsigned)((k + k_per - 1) / k_per));
@@ -1537,7 +1547,7 @@ static bool big_tile_pays(int m, int n, int k) {
 }
 
 template <typename TOut>
-static int launch_bf16(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k, int epilogue,
+static int launch_bf16(const bf16_t* x, const bf16_t* w, const float* bias, TOut* y, int m, int n, int k, Epilogue epilogue,
                        int force, int slices, hipStream_t s) {
     // `force` (for measurements): 1 = K-split kernel, 2/4/8 = shared activations with that many waves
     // 452: the 128 by 128 tile on four stages, at any number of rows
@@ -1602,7 +1612,7 @@ static int launch_bf16(const bf16_t* x, const bf16_t* w, const float* bias, TOut
 // 256 / 128, 452 the 128 by 128 tile on four stages, 351 / 451 the 128 by 64 tile on two / four stages;
 // with a variant, any number of K slices is taken.
 static int gemm_variant(const void* x, const void* w, const float* bias, void* y, int dtype, int out_dtype,
-                        int m, int n, int k, int epilogue, int slices, int variant, imparo_stream stream) {
+                        int m, int n, int k, Epilogue epilogue, int slices, int variant, imparo_stream stream) {
     if (!x || !w || !y || m < 0 || n <= 0 || k <= 0) return IMPARO_BAD_ARGUMENT;
     if (slices < 1) return IMPARO_BAD_ARGUMENT;
     // slices: only what imparo_gemm_slices allows, float32 out, no epilogue that is not linear
@@ -1652,6 +1662,11 @@ static int gemm_variant(const void* x, const void* w, const float* bias, void* y
 extern "C" int imparo_gemm(const void* x, const void* w, const float* bias, void* y, int dtype, int out_dtype,
                            int m, int n, int k, int epilogue, int slices, imparo_stream stream) {
     return gemm_variant(x, w, bias, y, dtype, out_dtype, m, n, k, epilogue, slices, 0, stream);
+}
+
+extern "C" int imparo_gemm_swiglu_scaled(const void* x, const void* w, const float* bias, void* y, int dtype, int out_dtype,
+                                         int m, int n, int k, float scale, imparo_stream stream) {
+    return gemm_variant(x, w, bias, y, dtype, out_dtype, m, n, k, Epilogue(EPI_SWIGLU, scale), 1, 0, stream);
 }
 
 extern "C" int imparo_gemm_variant(const void* x, const void* w, const float* bias, void* y, int dtype, int out_dtype,

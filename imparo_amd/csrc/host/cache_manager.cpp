@@ -74,6 +74,7 @@ struct Request {
 struct ImparoCache {
     int page_size;
     std::vector<int> windows;                            // 0 = every position; w > 0: the last w; w < 0: chunks of -w
+    std::vector<int> keep_pages;                         // pages from the start on that stay whatever the window
     std::vector<ImparoPool> pools;
     ImparoPool slots;
     std::unordered_map<int64_t, Request> live;
@@ -82,6 +83,7 @@ struct ImparoCache {
         : page_size(ps), slots(n_slots) {
         for (int g = 0; g < n_groups; ++g) {
             windows.push_back(w ? w[g] : 0);
+            keep_pages.push_back(0);
             pools.emplace_back(n_pages[g]);          // every group has a pool of its own size
         }
     }
@@ -131,6 +133,14 @@ ImparoCache* imparo_cache_new(int n_groups, const int32_t* windows, int page_siz
     return new ImparoCache(n_groups, windows, page_size, n_pages, n_slots);
 }
 void imparo_cache_delete(ImparoCache* c) { delete c; }
+// The first `n_tokens` positions of every request are read by all later ones: their pages are kept
+// although the group's window passes them.
+int imparo_cache_keep_first(ImparoCache* c, int group, int n_tokens) {
+    if (group < 0 || group >= (int)c->pools.size() || n_tokens < 0) return IMPARO_E_RANGE;
+    if (!c->live.empty()) return IMPARO_E_BUSY;
+    c->keep_pages[(size_t)group] = (int)(((int64_t)n_tokens + c->page_size - 1) / c->page_size);
+    return 0;
+}
 ImparoPool* imparo_cache_group_pool(ImparoCache* c, int group) {
     return (group < 0 || group >= (int)c->pools.size()) ? nullptr : &c->pools[(size_t)group];
 }
@@ -169,7 +179,7 @@ int imparo_cache_reserve(ImparoCache* c, int64_t req, int new_length) {
         const int first = c->first_needed_page((int)g, r.length);
         while ((int)table.size() < total) {
             int32_t page = -1;                                  // wholly behind the window: never needed
-            if ((int)table.size() >= first) {
+            if ((int)table.size() >= first || (int)table.size() < c->keep_pages[g]) {
                 page = c->pools[g].alloc();
                 if (page < 0) {                                 // undo what this call took, nothing else
                     while (r.pending.size() > mark) {
@@ -205,7 +215,7 @@ int imparo_cache_commit(ImparoCache* c, int64_t req, int new_length) {
         if (c->windows[g] == 0) continue;
         std::vector<int32_t>& table = r.tables[g];
         const int upto = std::min(c->first_needed_page((int)g, new_length), (int)table.size());
-        for (int i = 0; i < upto; ++i)
+        for (int i = c->keep_pages[g]; i < upto; ++i)
             if (table[(size_t)i] >= 0) {
                 c->pools[g].free_page(table[(size_t)i]);
                 table[(size_t)i] = -1;

@@ -64,6 +64,7 @@ int imparo_cache_slot(const ImparoCache* c, int64_t req);
 int imparo_cache_table_len(const ImparoCache* c, int group, int64_t req);
 int imparo_cache_table_copy(const ImparoCache* c, int group, int64_t req, int32_t* out, int capacity);
 int imparo_cache_pages_needed(const ImparoCache* c, int64_t req, int new_length, int32_t* per_group);
+int imparo_cache_keep_first(ImparoCache* c, int group, int n_tokens);
 int imparo_cache_first_needed_page(const ImparoCache* c, int group, int next_position);
 int imparo_cache_n_live(const ImparoCache* c);
 int imparo_cache_page_size(const ImparoCache* c);

@@ -38,6 +38,115 @@ extern "C" int imparo_embed_sinusoid(const void* table, int table_dtype, const i
     return launch_status();
 }
 
+// ---------------------------------------------------------------- a norm without a statistic
+// out = tanh(alpha v) w + b over the elements of a row, v = x + what is pending on it. Nothing crosses elements, so
+// a thread takes V neighbouring elements (4 where the width allows) and every load of it is asked for before any
+// is used.
+template <int V>
+struct RowPiece {
+    float e[V];
+};
+template <int V>
+__device__ __forceinline__ RowPiece<V> load_piece(const float* p) {
+    RowPiece<V> r;
+    if constexpr (V == 4) {
+        const float4 f = *reinterpret_cast<const float4*>(p);
+        r.e[0] = f.x, r.e[1] = f.y, r.e[2] = f.z, r.e[3] = f.w;
+    } else {
+#pragma unroll
+        for (int j = 0; j < V; ++j) r.e[j] = p[j];
+    }
+    return r;
+}
+// The slices of a delta, in order, four loads under way at once from clamped addresses.
+template <int V>
+__device__ __forceinline__ void add_slices(RowPiece<V>& d, const float* __restrict__ delta, int n, size_t stride, size_t at) {
+    for (int s0 = 0; s0 < n; s0 += 4) {
+        RowPiece<V> p[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) p[j] = load_piece<V>(delta + (size_t)min(s0 + j, n - 1) * stride + at);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int i = 0; i < V; ++i) d.e[i] += s0 + j < n ? p[j].e[i] : 0.f;
+    }
+}
+
+template <typename TOut, int V>
+__global__ void k_dynamic_tanh(float* __restrict__ x, const float* __restrict__ da, int n_a, const float* __restrict__ db,
+                               int n_b, size_t stride, const int32_t* __restrict__ rows, float alpha,
+                               const float* __restrict__ weight, const float* __restrict__ bias, TOut* __restrict__ out,
+                               int n_rows, int width, int write_back) {
+    const int per_row = width / V;
+    const long long id = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (id >= (long long)n_rows * per_row) return;
+    const int i_out = (int)(id / per_row), c = (int)(id - (long long)i_out * per_row) * V;
+    const size_t at = (size_t)(rows ? rows[i_out] : i_out) * width + c;
+    RowPiece<V> v = load_piece<V>(x + at);
+    const RowPiece<V> w = load_piece<V>(weight + c), b = load_piece<V>(bias + c);
+    if (n_a) {
+        RowPiece<V> d{};
+        add_slices<V>(d, da, n_a, stride, at);
+        if (n_b) {
+            RowPiece<V> e{};
+            add_slices<V>(e, db, n_b, stride, at);
+#pragma unroll
+            for (int j = 0; j < V; ++j) d.e[j] += e.e[j];
+        }
+#pragma unroll
+        for (int j = 0; j < V; ++j) v.e[j] += d.e[j];
+        if (write_back) {
+            if constexpr (V == 4) {
+                *reinterpret_cast<float4*>(x + at) = make_float4(v.e[0], v.e[1], v.e[2], v.e[3]);
+            } else {
+#pragma unroll
+                for (int j = 0; j < V; ++j) x[at + j] = v.e[j];
+            }
+        }
+    }
+    float y[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) y[j] = fmaf(tanhf(alpha * v.e[j]), w.e[j], b.e[j]);
+    const size_t dst = (size_t)i_out * width + c;
+    if constexpr (V == 4 && sizeof(TOut) == 2) {
+        *reinterpret_cast<uint2*>(out + dst) = make_uint2(f32x2_to_bf16x2(y[0], y[1]), f32x2_to_bf16x2(y[2], y[3]));
+    } else if constexpr (V == 4) {
+        *reinterpret_cast<float4*>(out + dst) = make_float4(y[0], y[1], y[2], y[3]);
+    } else {
+#pragma unroll
+        for (int j = 0; j < V; ++j) store_f32<TOut>(out, dst + j, y[j]);
+    }
+}
+
+extern "C" int imparo_dynamic_tanh(float* x, const float* delta_a, int n_a, const float* delta_b, int n_b, int n_x_rows,
+                                   const int32_t* rows, float alpha, const float* weight, const float* bias, void* out,
+                                   int out_dtype, int n_rows, int width, int write_back, imparo_stream stream) {
+    if (!x || !weight || !bias || !out || n_rows < 0 || width <= 0 || n_x_rows < 0) return IMPARO_BAD_ARGUMENT;
+    if (n_a < 0 || n_b < 0 || (n_a && !delta_a) || (n_b && !delta_b) || (n_b && !n_a)) return IMPARO_BAD_ARGUMENT;
+    if (write_back && rows) return IMPARO_BAD_ARGUMENT;
+    if (out_dtype != IMPARO_F32 && out_dtype != IMPARO_BF16) return IMPARO_BAD_ARGUMENT;
+    if (n_rows == 0) return IMPARO_OK;
+    hipStream_t s = (hipStream_t)stream;
+    const size_t stride = (size_t)n_x_rows * width;
+    const bool four = width % 4 == 0 && !(((uintptr_t)x | (uintptr_t)delta_a | (uintptr_t)delta_b | (uintptr_t)weight |
+                                           (uintptr_t)bias | (uintptr_t)out) & 15);
+    const long long n = (long long)n_rows * (four ? width / 4 : width);
+    const int threads = n <= 16384 ? 64 : 256;                  // few rows: over more CUs
+    const unsigned blocks = (unsigned)((n + threads - 1) / threads);
+#define DYN_TANH(T, V)                                                                                               \
+    k_dynamic_tanh<T, V><<<blocks, threads, 0, s>>>(x, delta_a, n_a, delta_b, n_b, stride, rows, alpha, weight, bias, \
+                                                    (T*)out, n_rows, width, write_back)
+    if (out_dtype == IMPARO_BF16) {
+        if (four) DYN_TANH(bf16_t, 4);
+        else DYN_TANH(bf16_t, 1);
+    } else {
+        if (four) DYN_TANH(float, 4);
+        else DYN_TANH(float, 1);
+    }
+#undef DYN_TANH
+    return launch_status();
+}
+
 // ---------------------------------------------------------------- RMS norm in groups
 // One block per output row, one wave per group at a time: the row is cut into `groups` equal
 // consecutive parts and each is divided by its own sqrt(mean(part^2) + eps); the whole is multiplied by

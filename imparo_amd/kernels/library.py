@@ -25,6 +25,8 @@ _SIGNATURES = {
     "imparo_place_tokens": [P, P, P, P, I, I, P],
     "imparo_rms_norm": [P, P, I, I, P, P, P, I, I, I, F, I, P],
     "imparo_gemm": [P, P, P, P, I, I, I, I, I, I, I, P],
+    # x, w, bias, y, dtype, out_dtype, m, n, k, scale, stream
+    "imparo_gemm_swiglu_scaled": [P, P, P, P, I, I, I, I, I, F, P],
     "imparo_gemm_slices": [I, I, I, I],
     "imparo_gemm_adds": [I, I, I, I],
     "imparo_gemm_variant": [P, P, P, P, I, I, I, I, I, I, I, I, P],
@@ -38,6 +40,11 @@ _SIGNATURES = {
     "imparo_attention_decode_qkv": [P, P, P, F, P, I, I, P, P, I, P, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P],
     "imparo_attention_decode_exact": [P, P, P, P, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P],
     "imparo_attention_prefill_exact": [P, P, P, P, P, P, I, P, I, I, P, P, P, P, I, I, I, I, I, I, F, I, P],
+    # as the exact forms, with the address of an AttentionRule before the stream
+    "imparo_attention_decode_ruled": [P, P, P, P, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P, P],
+    "imparo_attention_prefill_ruled": [P, P, P, P, P, P, I, P, I, I, P, P, P, P, I, I, I, I, I, I, F, I, P, P],
+    "imparo_attention_ruled": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, I, F, I, I, P, P],
+    "imparo_attention_ruled_keys": [I, I, I],
     "imparo_attention_decode_qkv_takes": [I, I],
     "imparo_attention_decode_qkv_pays": [I, I],
     "imparo_attention_prefill": [P, P, P, P, P, P, I, P, I, I, P, P, P, P, I, I, I, I, I, I, F, I, P],
@@ -82,13 +89,21 @@ _SIGNATURES = {
     "imparo_hgrn2_scan": [P, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, P, P, P],
     # q, ld, off, div, k, ld, off, div, v, ld, off, decay_const, step, ld, off, step_bias, rate, v_times_step, beta, ld,
     # off, skip, state, seg_start, seg_len, slot, out, n_rows, heads, dim, vdim, chunk_tokens, max_chunks, chunk_state,
-    # chunk_decay, stream
+    # chunk_decay, silu_in, stream
     "imparo_decay_scan": [P, I, I, I, P, I, I, I, P, I, I, P, P, I, I, P, P, I, P, I, I, P, P, P, P, P, P, I, I, I, I, I, I,
-                          P, P, P],
+                          P, P, I, P],
+    # q, ld, off, div, k, ld, off, div, v, ld, off, step, ld, off, step_bias, rate, beta, ld, off, state, seg_start,
+    # seg_len, slot, out, n_rows, heads, dim, vdim, chunk_tokens, max_chunks, scratch, stream
+    "imparo_channel_delta_scan": [P, I, I, I, P, I, I, I, P, I, I, P, I, I, P, P, P, I, I, P, P, P, P, P, I, I, I, I, I, I,
+                                  P, P],
+    "imparo_channel_delta_scratch": ([I], c_int64),
+    "imparo_silu_columns": [P, I, I, I, I, P],
+    # x, delta_a, n_a, delta_b, n_b, n_x_rows, rows, alpha, weight, bias, out, out_dtype, n_rows, width, write_back, stream
+    "imparo_dynamic_tanh": [P, P, I, P, I, I, P, F, P, P, P, I, I, I, I, P],
     "imparo_delta_chunk_tokens": [],
     "imparo_delta_chunk_max_dim": [],
     "imparo_head_prepare": [P, I, I, I, I, I, I, F, P, I, I, P, I, F, F, P],
-    "imparo_gated_group_norm": [P, P, I, I, P, P, I, I, I, I, F, I, P],
+    "imparo_gated_group_norm": [P, P, I, I, P, P, I, I, I, I, F, I, I, P],
     "imparo_clamped_glu": [P, P, I, I, I, I, F, F, P],
     "imparo_normed_sum": [P, I, P, P, I, P, P, I, I, F, F, P],
     "imparo_gated_row_add": [P, P, I, P, I, I, I, I, P],

@@ -111,6 +111,31 @@ def place_tokens(ids: torch.Tensor, dst: torch.Tensor, src: torch.Tensor, src_in
     return ids
 
 
+def dynamic_tanh(x: torch.Tensor, alpha: float, weight: torch.Tensor, bias: torch.Tensor, out: torch.Tensor,
+                 deltas=(), rows: Optional[torch.Tensor] = None, write_back: bool = False) -> torch.Tensor:
+    """out[i] = tanh(alpha v) * weight + bias, v = x[src] + the pending deltas' rows (up to two, each shaped like x or
+    [slices, *x.shape]), src = rows[i] or i. write_back stores v into x (only without rows)."""
+    n_x, width = x.shape
+    n_out = out.shape[0]
+    if (rows is None and n_out != n_x) or (rows is not None and rows.shape[0] != n_out):
+        raise KernelArgumentError("dynamic_tanh: one source row per output row is needed")
+    if write_back and (rows is not None or not deltas):
+        raise KernelArgumentError("dynamic_tanh: write_back needs a delta and no row selection")
+    if len(deltas) > 2:
+        raise KernelArgumentError(f"dynamic_tanh: up to two deltas are added, got {len(deltas)}")
+    args = []
+    for d in tuple(deltas) + (None,) * (2 - len(deltas)):
+        slices = 0 if d is None else d.shape[0] if d.dim() == 3 else 1
+        args += [_dev(d, "delta", torch.float32, None if d is None else (slices, n_x, width) if d.dim() == 3 else (n_x, width)),
+                 slices]
+    _check(library().imparo_dynamic_tanh(
+        _dev(x, "stream", torch.float32), *args, n_x, _dev(rows, "rows", torch.int32), float(alpha),
+        _dev(weight, "norm weight", torch.float32, (width,)), _dev(bias, "norm bias", torch.float32, (width,)),
+        _dev(out, "normed", None, (n_out, width)), _code(out, "normed"), n_out, width, int(write_back), _stream()),
+        "dynamic_tanh")
+    return out
+
+
 def rms_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor,
              delta: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None,
              write_back: bool = False) -> torch.Tensor:
@@ -149,10 +174,10 @@ def gemm_adds(m: int, n: int, k: int, dtype: torch.dtype) -> bool:
 
 
 def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None,
-         swiglu: bool = False, variant: int = 0, add: bool = False) -> torch.Tensor:
+         swiglu: bool = False, variant: int = 0, add: bool = False, swiglu_scale: float = 1.0) -> torch.Tensor:
     """out[m, n] = x[m, k] . w[n, k]^T (+ bias[n]); x and w share a dtype; float32
     accumulate. With `swiglu` the rows of w alternate gate and up and out is
-    [m, n/2] = silu(gate) * up. An `out` of shape [slices, m, n] (slices =
+    [m, n/2] = silu(gate) * up (* swiglu_scale, before it is rounded). An `out` of shape [slices, m, n] (slices =
     gemm_slices(...)) receives the sums over slices of K, to be added by the consumer.
     With `add` (float32 out, where gemm_adds(...) says so) the product is added to what `out` holds.
     `variant` other than 0 names the kernel (tests and measurements only; see imparo_gemm_variant)."""
@@ -178,7 +203,11 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[tor
         raise KernelArgumentError("gemm: this product cannot be added to what its output holds")
     args = (_dev(x, "gemm x"), _dev(w, "gemm weight"), _dev(bias, "gemm bias", torch.float32, (n,)),
             out.data_ptr(), _code(x, "gemm x"), _code(out, "gemm out"), m, n, k, 2 if add else int(swiglu), slices)
-    if variant:
+    if swiglu_scale != 1.0:
+        if not swiglu or variant:
+            raise KernelArgumentError("gemm: a scale goes with the gated epilogue only")
+        _check(library().imparo_gemm_swiglu_scaled(*args[:9], float(swiglu_scale), _stream()), "gemm")
+    elif variant:
         _check(library().imparo_gemm_variant(*args, int(variant), _stream()), "gemm")
     else:
         _check(library().imparo_gemm(*args, _stream()), "gemm")
@@ -222,9 +251,37 @@ def qk_norm_rope_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_we
     return q_out
 
 
+class AttentionRule(ctypes.Structure):
+    """What a layer's attention asks for beyond a window: `keep_first` (so many positions from the start stay visible),
+    `softcap` (0: none), `sink` (address of one float32 a head, or null), `out_scale` (a factor on the result)."""
+    _fields_ = [("keep_first", ctypes.c_int), ("softcap", ctypes.c_float), ("sink", ctypes.c_void_p),
+                ("out_scale", ctypes.c_float)]
+
+
+def attention_rule(heads: int, keep_first: int = 0, softcap: Optional[float] = None, sink: Optional[torch.Tensor] = None,
+                   out_scale: float = 1.0) -> AttentionRule:
+    """The rule for a layer of `heads` heads; it keeps the sink's tensor alive."""
+    rule = AttentionRule(int(keep_first), float(softcap or 0.0), _dev(sink, "sinks", torch.float32, (heads,)) or None,
+                         float(out_scale))
+    rule.heads, rule.held = heads, sink
+    return rule
+
+
+def _rule(rule: AttentionRule, heads: int):
+    if rule.heads != heads:
+        raise KernelArgumentError(f"attention: a rule for {rule.heads} heads was given to a layer of {heads}")
+    return ctypes.addressof(rule)
+
+
+def attention_ruled_keys(max_context: int, window: Optional[int], rule: AttentionRule) -> int:
+    """The most keys a query below `max_context` walks over under this window and rule."""
+    return int(library().imparo_attention_ruled_keys(int(max_context), int(window or 0), int(rule.keep_first)))
+
+
 def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, out: torch.Tensor,
               positions: torch.Tensor, row_of_token: torch.Tensor, block_table: torch.Tensor,
-              scale: float, window: Optional[int], v_transposed: bool = False) -> torch.Tensor:
+              scale: float, window: Optional[int], v_transposed: bool = False,
+              rule: Optional[AttentionRule] = None) -> torch.Tensor:
     """The general kernel: any page size, head sizes up to 512 (values of a size of their own
     are read off the value cache's shape), float32 or bfloat16; one wave per (token, head). `out`
     may be wider than heads x value size: the rest of a row is written as zeros."""
@@ -237,7 +294,7 @@ def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, out
         raise KernelArgumentError(f"attention: {heads} heads cannot share {kv_heads} kv heads evenly")
     if out.dim() != 2 or out.shape[0] != n or out.shape[1] < heads * value_dim:
         raise KernelArgumentError(f"attention: out is {list(out.shape)}; [{n}, at least {heads * value_dim}] is needed")
-    _check(library().imparo_attention_dv(
+    args = (
         _dev(q, "q"), _dev(k_cache, "k cache", q.dtype),
         _dev(v_cache, "v cache", q.dtype, (n_pages, kv_heads, value_dim, page_size) if v_transposed
              else (n_pages, kv_heads, page_size, value_dim)),
@@ -245,7 +302,11 @@ def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, out
         _dev(positions, "positions", torch.int32, (n,)), _dev(row_of_token, "row_of_token", torch.int32, (n,)),
         _dev(block_table, "block table", torch.int32), block_table.shape[1], page_size,
         n, heads, kv_heads, head_dim, value_dim, out.shape[1], n_pages, float(scale), int(window or 0),
-        int(v_transposed), _stream()), "attention")
+        int(v_transposed))
+    if rule is not None:
+        _check(library().imparo_attention_ruled(*args, _rule(rule, heads), _stream()), "attention")
+    else:
+        _check(library().imparo_attention_dv(*args, _stream()), "attention")
     return out
 
 
@@ -281,22 +342,32 @@ def _check_mfma(q, k_cache, v_cache, out):
 
 def attention_decode(q, k_cache, v_cache, out, part_o, part_ml, rows, n_rows: int, seg_start, positions,
                      block_table, scale: float, window: Optional[int], max_context: int,
-                     exact: bool = False) -> torch.Tensor:
+                     exact: bool = False, rule: Optional[AttentionRule] = None) -> torch.Tensor:
     """Split-KV attention for rows that bring one token each. `rows` lists
     them (indices into seg_start); `max_context` bounds every row's position + 1.
-    `exact`: the softmax weights keep float32's precision through the product with the values."""
+    `exact`: the softmax weights keep float32's precision through the product with the values. `rule` (with `exact`):
+    splits are counted over the keys a query can see (attention_ruled_keys)."""
     n, heads, head_dim, n_pages, kv_heads, page_size = _check_mfma(q, k_cache, v_cache, out)
     split = decode_split()
+    if rule is not None:
+        if not exact:
+            raise KernelArgumentError("attention_decode: a rule goes with exact weights")
+        max_context = attention_ruled_keys(max_context, window, rule)
     n_splits = max(1, (max_context + split - 1) // split)
     if part_o.numel() < n_rows * heads * n_splits * head_dim or part_ml.numel() < n_rows * heads * n_splits * 2:
         raise KernelArgumentError("attention_decode: the scratch for partial results is too small")
-    _check((library().imparo_attention_decode_exact if exact else library().imparo_attention_decode)(
+    args = (
         _dev(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(),
         _dev(part_o, "partial outputs", torch.float32), _dev(part_ml, "partial sums", torch.float32),
         _dev(rows, "decode rows", torch.int32), n_rows, _dev(seg_start, "seg_start", torch.int32),
         _dev(positions, "positions", torch.int32, (n,)), _dev(block_table, "block table", torch.int32),
         block_table.shape[1], page_size, heads, kv_heads, head_dim, n_pages, float(scale), int(window or 0),
-        n_splits, _stream()), "attention_decode")
+        n_splits)
+    if rule is not None:
+        _check(library().imparo_attention_decode_ruled(*args, _rule(rule, heads), _stream()), "attention_decode")
+    else:
+        _check((library().imparo_attention_decode_exact if exact else library().imparo_attention_decode)(*args, _stream()),
+               "attention_decode")
     return out
 
 
@@ -353,7 +424,8 @@ def attention_prefill_splits(n_tiles: int, heads: int, kv_heads: int, head_dim: 
 
 def attention_prefill(q, k_cache, v_cache, out, rows, n_rows: int, n_tiles: int, seg_start, seg_len, positions,
                       block_table, scale: float, window: Optional[int], part_o: Optional[torch.Tensor] = None,
-                      part_ml: Optional[torch.Tensor] = None, n_splits: int = 1, exact: bool = False) -> torch.Tensor:
+                      part_ml: Optional[torch.Tensor] = None, n_splits: int = 1, exact: bool = False,
+                      rule: Optional[AttentionRule] = None) -> torch.Tensor:
     """Tiled attention for rows that bring a portion of a prompt. `n_tiles` is
     the sum over the listed rows of ceil(seg_len / prefill_tile()). With `n_splits` > 1
     (attention_prefill_splits) each block's keys are walked in that many parts,
@@ -367,13 +439,20 @@ def attention_prefill(q, k_cache, v_cache, out, rows, n_rows: int, n_tiles: int,
         _dev(part_ml, "part_ml", torch.float32)
         if part_o.numel() < n * heads * n_splits * head_dim or part_ml.numel() < n * heads * n_splits * 2:
             raise KernelArgumentError("attention_prefill: the buffers for the parts are too small")
-    _check((library().imparo_attention_prefill_exact if exact else library().imparo_attention_prefill)(
+    if rule is not None and not exact:
+        raise KernelArgumentError("attention_prefill: a rule goes with exact weights")
+    args = (
         _dev(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), out.data_ptr(),
         part_o.data_ptr() if n_splits > 1 else None, part_ml.data_ptr() if n_splits > 1 else None, int(n_splits),
         _dev(rows, "prefill rows", torch.int32), n_rows, n_tiles, _dev(seg_start, "seg_start", torch.int32),
         _dev(seg_len, "seg_len", torch.int32), _dev(positions, "positions", torch.int32, (n,)),
         _dev(block_table, "block table", torch.int32), block_table.shape[1], page_size, heads, kv_heads, head_dim,
-        n_pages, float(scale), int(window or 0), _stream()), "attention_prefill")
+        n_pages, float(scale), int(window or 0))
+    if rule is not None:
+        _check(library().imparo_attention_prefill_ruled(*args, _rule(rule, heads), _stream()), "attention_prefill")
+    else:
+        _check((library().imparo_attention_prefill_exact if exact else library().imparo_attention_prefill)(*args, _stream()),
+               "attention_prefill")
     return out
 
 
@@ -1170,13 +1249,15 @@ def decay_scan(q: torch.Tensor, q_off: int, q_div: int, k: torch.Tensor, k_off: 
                step: Optional[torch.Tensor] = None, step_off: int = 0, step_bias: Optional[torch.Tensor] = None,
                rate: Optional[torch.Tensor] = None, v_times_step: bool = False, beta: Optional[torch.Tensor] = None,
                beta_off: int = 0, skip: Optional[torch.Tensor] = None, chunk_tokens: int = 0, max_chunks: int = 1,
-               chunk_state: Optional[torch.Tensor] = None, chunk_decay: Optional[torch.Tensor] = None) -> torch.Tensor:
+               chunk_state: Optional[torch.Tensor] = None, chunk_decay: Optional[torch.Tensor] = None,
+               silu_in: bool = False) -> torch.Tensor:
     """Per request, head and token in order: S <- a S + k v^T, out = S^T q; with `beta` the gated delta rule
     S <- a S, u = sigmoid(beta) (v - S^T k), S <- S + k u^T, out = S^T q. q, k, v, step, beta are float32 row
     tensors [tokens, ld] read from a column offset on (they may be one tensor); head h reads q head h // q_div
     and k head h // k_div. a = decay_const[h] or exp(-rate[h] softplus(step[t, h] + step_bias[h])); with
     `v_times_step` v is multiplied by that softplus; with `skip`, out += skip[h] v. state [slots, heads, dim,
-    vdim] float32 is carried on; out [tokens, heads * vdim] float32."""
+    vdim] float32 is carried on; out [tokens, heads * vdim] float32. `silu_in`: q, k and v go through SiLU as they
+    are read (token by token and without `beta` only)."""
     n = out.shape[0]
     n_rows = seg_start.shape[0]
     if dim > DECAY_SCAN_MAX_DIM:
@@ -1184,6 +1265,8 @@ def decay_scan(q: torch.Tensor, q_off: int, q_div: int, k: torch.Tensor, k_off: 
     for t, what in ((q, "q"), (k, "k"), (v, "v"), (step, "step"), (beta, "beta")):
         if t is not None and (t.dim() != 2 or t.shape[0] != n):
             raise KernelArgumentError(f"decay_scan: {what} is not a row tensor of {n} tokens")
+    if silu_in and (chunk_tokens or beta is not None):
+        raise KernelArgumentError("decay_scan: SiLU on the way in is for the plain recurrence token by token")
     if (decay_const is None) == (step is None):
         raise KernelArgumentError("decay_scan: the decay is a constant a head or comes from projected steps")
     if chunk_tokens:
@@ -1205,8 +1288,63 @@ def decay_scan(q: torch.Tensor, q_off: int, q_div: int, k: torch.Tensor, k_off: 
         _dev(slot, "slot", torch.int32, (n_rows,)), _dev(out, "scan out", torch.float32, (n, heads * vdim)),
         n_rows, heads, dim, vdim, int(chunk_tokens), int(max_chunks),
         _dev(chunk_state, "chunk states", torch.float32) if chunk_tokens else 0,
-        _dev(chunk_decay, "chunk decays", torch.float32) if chunk_tokens else 0, _stream()), "decay_scan")
+        _dev(chunk_decay, "chunk decays", torch.float32) if chunk_tokens else 0, int(bool(silu_in)), _stream()), "decay_scan")
     return out
+
+
+def channel_delta_chunks(max_seg_len: int, dim: int):
+    """(chunk_tokens, max_chunks) for `channel_delta_scan`: (0, 1), token by token, for short segments and wide heads."""
+    chunk = int(library().imparo_delta_chunk_tokens())
+    if dim > int(library().imparo_delta_chunk_max_dim()) or max_seg_len < 2 * chunk:
+        return 0, 1
+    return chunk, -(-int(max_seg_len) // chunk)
+
+
+def channel_delta_scratch(n_rows: int, max_chunks: int, heads: int, dim: int) -> int:
+    """Floats of scratch that `channel_delta_scan` needs when it walks in chunks."""
+    return n_rows * max_chunks * heads * int(library().imparo_channel_delta_scratch(dim))
+
+
+def channel_delta_scan(q: torch.Tensor, q_off: int, q_div: int, k: torch.Tensor, k_off: int, k_div: int, v: torch.Tensor,
+                       v_off: int, step: torch.Tensor, step_off: int, step_bias: torch.Tensor, rate: torch.Tensor,
+                       beta: torch.Tensor, beta_off: int, state: torch.Tensor, seg_start: torch.Tensor,
+                       seg_len: torch.Tensor, slot: torch.Tensor, out: torch.Tensor, heads: int, dim: int, vdim: int,
+                       chunk_tokens: int = 0, max_chunks: int = 1, scratch: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Per request, head and token in order the gated delta rule with one decay a state row: S <- diag(g) S,
+    u = sigmoid(beta) (v - S^T k), S <- S + k u^T, out = S^T q, g = exp(-rate[h] softplus(step[t, h dim + i] +
+    step_bias[h dim + i])). q, k, v, step, beta are float32 row tensors read from a column offset on; head h reads q
+    head h // q_div and k head h // k_div. state [slots, heads, dim, vdim] float32 is carried on."""
+    n = out.shape[0]
+    n_rows = seg_start.shape[0]
+    if dim > DECAY_SCAN_MAX_DIM:
+        raise KernelArgumentError(f"channel_delta_scan: up to {DECAY_SCAN_MAX_DIM} state rows a head, got {dim}")
+    for t, what in ((q, "q"), (k, "k"), (v, "v"), (step, "step"), (beta, "beta")):
+        if t.dim() != 2 or t.shape[0] != n:
+            raise KernelArgumentError(f"channel_delta_scan: {what} is not a row tensor of {n} tokens")
+    if chunk_tokens and (scratch is None or scratch.numel() < channel_delta_scratch(n_rows, max_chunks, heads, dim)):
+        raise KernelArgumentError("channel_delta_scan: the scratch for the chunks is too small")
+    _check(library().imparo_channel_delta_scan(
+        _dev(q, "scan q", torch.float32), q.shape[1], int(q_off), int(q_div),
+        _dev(k, "scan k", torch.float32), k.shape[1], int(k_off), int(k_div),
+        _dev(v, "scan v", torch.float32), v.shape[1], int(v_off),
+        _dev(step, "steps", torch.float32), step.shape[1], int(step_off),
+        _dev(step_bias, "step bias", torch.float32, (heads * dim,)), _dev(rate, "decay rates", torch.float32, (heads,)),
+        _dev(beta, "beta", torch.float32), beta.shape[1], int(beta_off),
+        _dev(state, "scan state", torch.float32, (state.shape[0], heads, dim, vdim)),
+        _dev(seg_start, "seg_start", torch.int32, (n_rows,)), _dev(seg_len, "seg_len", torch.int32, (n_rows,)),
+        _dev(slot, "slot", torch.int32, (n_rows,)), _dev(out, "scan out", torch.float32, (n, heads * vdim)),
+        n_rows, heads, dim, vdim, int(chunk_tokens), int(max_chunks),
+        _dev(scratch, "chunk scratch", torch.float32) if chunk_tokens else 0, _stream()), "channel_delta_scan")
+    return out
+
+
+def silu_columns(rows: torch.Tensor, off: int, n: int) -> torch.Tensor:
+    """SiLU in place on columns off .. off + n - 1 of float32 rows."""
+    if off < 0 or n < 1 or off + n > rows.shape[1]:
+        raise KernelArgumentError(f"silu_columns: columns {off}..{off + n - 1} of rows of {rows.shape[1]}")
+    _check(library().imparo_silu_columns(_dev(rows, "rows", torch.float32), rows.shape[1], int(off), int(n), rows.shape[0],
+                                         _stream()), "silu_columns")
+    return rows
 
 
 def head_prepare(rows: torch.Tensor, off: int, heads: int, dim: int, unit: bool = False, unit_eps: float = 0.0,
@@ -1229,9 +1367,12 @@ def head_prepare(rows: torch.Tensor, off: int, heads: int, dim: int, unit: bool 
     return rows
 
 
+GATE_ACTS = {"silu": 0, "sigmoid": 1}
+
+
 def gated_group_norm(x: torch.Tensor, gate: Optional[torch.Tensor], gate_off: int, weight: Optional[torch.Tensor],
-                     groups: int, eps: float, out: torch.Tensor, gate_first: bool) -> torch.Tensor:
-    """A row of x (float32 [tokens, width]) in `groups` equal parts, g = silu(gate[t, gate_off + c]):
+                     groups: int, eps: float, out: torch.Tensor, gate_first: bool, gate_act: str = "silu") -> torch.Tensor:
+    """A row of x (float32 [tokens, width]) in `groups` equal parts, g = silu(gate[t, gate_off + c]), or its sigmoid:
     gate_first: (x g) / rms_part(x g) * weight; otherwise x / rms_part(x) * weight * g. weight [width] or None."""
     n, width = x.shape
     if gate is not None and (gate.dim() != 2 or gate.shape[0] != n or gate_off + width > gate.shape[1]):
@@ -1239,7 +1380,7 @@ def gated_group_norm(x: torch.Tensor, gate: Optional[torch.Tensor], gate_off: in
     _check(library().imparo_gated_group_norm(
         _dev(x, "heads' results", torch.float32), _dev(gate, "gate", torch.float32), 0 if gate is None else gate.shape[1],
         int(gate_off), _dev(weight, "norm weight", torch.float32, (width,)), _dev(out, "normed", None, (n, width)),
-        _code(out, "normed"), n, width, int(groups), float(eps), int(bool(gate_first)), _stream()), "gated_group_norm")
+        _code(out, "normed"), n, width, int(groups), float(eps), int(bool(gate_first)), GATE_ACTS[gate_act], _stream()), "gated_group_norm")
     return out
 
 

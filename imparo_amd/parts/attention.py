@@ -24,7 +24,14 @@ projected rows of a request are state beside its pages),
 `exact_weights` (the softmax weights keep float32's precision through the
 product with the values: the matrix-core kernels then send what rounding a
 weight to bfloat16 took off through a second product; the wave kernel, which
-takes every other shape, keeps its weights in float32 anyway)."""
+takes every other shape, keeps its weights in float32 anyway),
+`keep_first` (beside its window a query sees the first so many positions,
+whose pages the cache keeps), `softcap` (a scaled score s becomes softcap *
+tanh(s / softcap)), `sink` (the name, under the prefix, of one learned number a
+head: the softmax's denominator holds one more term, its exponential, which
+belongs to no key), `out_scale` (a factor on the mixer's result: the attention
+rows carry it, in float32 before they are rounded). The last three and
+keep_first run with exact weights."""
 from __future__ import annotations
 
 from typing import Dict, Optional
@@ -68,6 +75,8 @@ class Attention:
             out[n["q_norm"] + sfx] = (TensorDecl((D,), "vector"), "norm")
             if not shared:
                 out[n["k_norm"] + sfx] = (TensorDecl((D,), "vector"), "norm")
+        if spec.get("sink"):
+            out[f"{spec.prefix}.{spec['sink']}"] = (TensorDecl((H,), "vector"), "wide")
         sides = ("q",) if shared else ("q", "k", "v")
         rows = dict(q=H * D, k=Hk * D, v=Hk * Dv)
         if spec.get("bias"):
@@ -101,6 +110,15 @@ class Attention:
             if self.window is not None or self.keep_window is not None or self.chunk < 1:
                 raise ValueError("a layer sees a window or its own chunk (of at least one position), not both")
             self.window = -int(self.chunk)        # as the kernels take it: a negative window is a chunk of that size
+        self.keep_first = int(spec.get("keep_first") or 0) if self.window is not None else 0
+        if self.keep_first and self.keep_window != self.window and self.chunk is None:
+            raise ValueError("first positions are kept beside the layer's own window")
+        sink = place_vector(tensors[f"{spec.prefix}.{spec['sink']}"], device) if spec.get("sink") else None
+        out_scale = float(spec.get("out_scale", 1.0))
+        self.rule = None          # None: the plain kernels
+        if self.keep_first or spec.get("softcap") or sink is not None or out_scale != 1.0:
+            self.rule = ops.attention_rule(self.heads, self.keep_first, spec.get("softcap"), sink, out_scale)
+            self.exact_weights = True
         sides = ("q",) if self.shared_kv else ("q", "k", "v")
         ws = [tensors[n[x] + sfx] for x in sides]
         if len({w.dtype for w in ws}) > 1:
@@ -155,7 +173,8 @@ class Attention:
         16, head sizes up to 128), V is kept transposed inside a page."""
         self.v_transposed = (self.value_dim == self.head_dim
                              and ops.mfma_attention_supported(self.engine_dtype, page_size, self.head_dim))
-        spec = kv_spec(self.kv_heads, self.head_dim, self.keep_window, self.v_transposed, self.value_dim, self.chunk)
+        spec = kv_spec(self.kv_heads, self.head_dim, self.keep_window, self.v_transposed, self.value_dim, self.chunk,
+                       self.keep_first)
         if self.conv_taps > 1:
             spec = with_fixed_arrays(spec, (FixedArray("conv", (self.conv_taps - 1, self.qkv.out_features), "float32", 0.0),))
         return spec
@@ -171,7 +190,8 @@ class Attention:
     def _decode_parts(self, ctx: StepContext):
         """Room for the partial results of the single-token rows' splits."""
         split = ops.decode_split()
-        n_splits = (ctx.max_context + split - 1) // split
+        keys = ctx.max_context if self.rule is None else ops.attention_ruled_keys(ctx.max_context, self.window, self.rule)
+        n_splits = (keys + split - 1) // split
         part_o = ctx.workspace.get("attn_part_o", (ctx.n_single_rows * self.heads * n_splits * self.head_dim,),
                                    torch.float32)
         part_ml = ctx.workspace.get("attn_part_ml", (ctx.n_single_rows * self.heads * n_splits * 2,), torch.float32)
@@ -219,13 +239,15 @@ class Attention:
                 part_o, part_ml = self._decode_parts(ctx)
                 ops.attention_decode(q, k_cache, v_cache, o, part_o, part_ml, ctx.single_rows, ctx.n_single_rows,
                                      ctx.seg_start, ctx.positions, table, self.scale, self.window, ctx.max_context,
-                                     exact=self.exact_weights)
+                                     exact=self.exact_weights, rule=self.rule)
             if ctx.n_portion_rows:
                 # few queries over long contexts: each block's keys in parts, merged by a second launch
                 n_tiles = self._portion_tiles(ctx)
                 # (the bound on the contexts that the launch itself sees: what its block table can hold)
-                parts = ops.attention_prefill_splits(n_tiles, self.heads, self.kv_heads, self.head_dim,
-                                                     table.shape[1] * ctx.page_size)
+                bound = table.shape[1] * ctx.page_size
+                if self.rule is not None:       # (a tile's 64 queries lie up to 64 positions apart)
+                    bound = ops.attention_ruled_keys(bound, self.window + 64 if (self.window or 0) > 0 else self.window, self.rule)
+                parts = ops.attention_prefill_splits(n_tiles, self.heads, self.kv_heads, self.head_dim, bound)
                 part_o = part_ml = None
                 if parts > 1:
                     part_o = ctx.workspace.get("attn_prefill_part_o", (T * self.heads * parts * self.head_dim,),
@@ -233,10 +255,11 @@ class Attention:
                     part_ml = ctx.workspace.get("attn_prefill_part_ml", (T * self.heads * parts * 2,), torch.float32)
                 ops.attention_prefill(q, k_cache, v_cache, o, ctx.portion_rows, ctx.n_portion_rows,
                                       n_tiles, ctx.seg_start, ctx.seg_len, ctx.positions, table,
-                                      self.scale, self.window, part_o, part_ml, parts, exact=self.exact_weights)
+                                      self.scale, self.window, part_o, part_ml, parts, exact=self.exact_weights,
+                                      rule=self.rule)
         else:
             ops.attention(q, k_cache, v_cache, o, ctx.positions, ctx.row_of_token, table, self.scale, self.window,
-                          v_transposed=vt)
+                          v_transposed=vt, rule=self.rule)
         if o.dtype != self.out.in_dtype:
             raise ValueError("the output projection's weight dtype differs from the attention output's")
         # a delta for the residual stream: the next norm adds slices, so it may come sliced

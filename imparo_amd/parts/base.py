@@ -147,12 +147,24 @@ class Residual:
     """The residual stream in float32 and a delta not yet added to it. The
     next norm adds the delta while it reads the row anyway. The delta is
     shaped like x, or [slices, *x.shape]: sums over parts of a projection's
-    inner dimension, which the norm adds up in order."""
+    inner dimension, which the norm adds up in order. Two mixers side by side
+    may leave a tuple of two such deltas."""
     x: torch.Tensor
     pending: Optional[torch.Tensor] = None
     # (weight, eps) of an RMS norm that the pending delta goes through before it is added (a block that
     # norms what its sublayers return); the norm that adds the delta applies it in the same launch
     post: Optional[Tuple[torch.Tensor, float]] = None
+
+
+def one_delta(res: Residual) -> None:
+    """For a reader that adds one delta: of a pending tuple all but the last are added to the stream now, slice by slice."""
+    if not isinstance(res.pending, tuple):
+        return
+    from ..kernels import ops
+    for d in res.pending[:-1]:
+        for part in (d if d.dim() == res.x.dim() + 1 else [d]):
+            ops.add_rows(res.x, part)
+    res.pending = res.pending[-1]
 
 
 @dataclass

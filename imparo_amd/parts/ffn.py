@@ -1,5 +1,7 @@
 """Dense SwiGLU feed-forward: f = W2 ( silu(W1 n) * (W3 n) ), SiLU on the gate
-(/root/reference/crates/imparo-model/src/lfm2/workflow_cpu.rs:298-316).
+(/root/reference/crates/imparo-model/src/lfm2/workflow_cpu.rs:298-316). `out_scale`
+multiplies f (a residual multiplier): the hidden values carry it, in float32
+before they are rounded.
 
 PolyNorm feed-forward: f = Wdown act(Wup n) with act(z) = a N(z) + b N(z^2) +
 c N(z^3) + e, powers taken element by element and N dividing a token's vector
@@ -49,6 +51,7 @@ class SwiGlu:
         self.width, self.hidden = spec["width"], spec["hidden"]
         # a second feed-forward inside another part keeps its scratch under names of its own
         self.tag = spec.get("scratch_tag") or ""
+        self.out_scale = float(spec.get("out_scale", 1.0))
         gate, up = tensors[n["gate"] + sfx], tensors[n["up"] + sfx]
         if gate.dtype != up.dtype:
             gate, up = gate.to(torch.float32), up.to(torch.float32)
@@ -73,13 +76,14 @@ class SwiGlu:
 
     def forward(self, ctx: StepContext, n: torch.Tensor) -> torch.Tensor:
         # the gated hidden may lie where the mixer's input projection lay: that is dead by now
-        g = self.gate_up(ctx, n, self.down.in_dtype, self.tag + "gated", swiglu=True, alias="mixer_in")
+        g = self.gate_up(ctx, n, self.down.in_dtype, self.tag + "gated", swiglu=True, alias="mixer_in",
+                         swiglu_scale=self.out_scale)
         # the result is a delta for the residual stream, whose next norm adds slices: it may come sliced
         return self.down(ctx, g, torch.float32, self.tag + "ffn_out", sliced_ok=True, into=ctx.stream)
 
 
     def can_emit(self) -> bool:
-        return not self.tag
+        return not self.tag and self.out_scale == 1.0
 
     def emit(self, program) -> None:
         """Appends `forward` to a native step program."""

@@ -2,7 +2,11 @@
 
 Both read the same h. Each result is divided by its root mean square over the
 model's width and multiplied by a weight of its own (plain, not one-plus), and
-the mixer's result is `factor` times their sum (one half unless given).
+the mixer's result is `factor` times their sum (one half unless given). With
+`normed` False there are no such norms and no factor: the result is the plain
+sum (what either side is multiplied by is that side's own `out_scale`), each
+side adds to the stream itself where it can, and what is left is handed on as
+one delta or two.
 
 The two are any registered mixers (`left`, `right`: their PartSpecs). What
 they keep between steps lives in one cache site: the pages of the one that
@@ -12,11 +16,12 @@ its own names through a view of the step's context, and the left one keeps its
 scratch under names of its own, since its result must outlive the right one's
 run.
 
-Parameters: width, eps, left, right, factor, names (left_out, right_out).
+Parameters: width, eps, left, right, factor, normed, names (left_out, right_out).
 """
 from __future__ import annotations
 
-from typing import Dict
+from dataclasses import replace
+from typing import Dict, Optional
 
 import torch
 
@@ -47,12 +52,13 @@ class _ScopedWorkspace:
 
 class _Scoped:
     """The step's context as one of the two mixers sees it: the site's fixed-size arrays that are
-    its own, under its own names; no stream to add into (the pair's result is made of both)."""
+    its own, under its own names; the stream to add into only where the pair's result is the plain sum."""
 
-    def __init__(self, ctx: StepContext, prefix: str, scratch_prefix: str = ""):
+    def __init__(self, ctx: StepContext, prefix: str, scratch_prefix: str = "",
+                 stream: Optional[torch.Tensor] = None):
         self._ctx, self._prefix = ctx, prefix
         self.workspace = _ScopedWorkspace(ctx.workspace, scratch_prefix) if scratch_prefix else ctx.workspace
-        self.stream = None
+        self.stream = stream
 
     def __getattr__(self, name):
         return getattr(self._ctx, name)
@@ -78,8 +84,10 @@ class MixerPair:
     @classmethod
     def declare(cls, spec: PartSpec) -> Declared:
         n = cls._names(spec)
-        out: Declared = {n["left_out"]: (TensorDecl((spec["width"],), "vector"), "norm"),
-                         n["right_out"]: (TensorDecl((spec["width"],), "vector"), "norm")}
+        out: Declared = {}
+        if spec.get("normed", True):
+            out = {n["left_out"]: (TensorDecl((spec["width"],), "vector"), "norm"),
+                   n["right_out"]: (TensorDecl((spec["width"],), "vector"), "norm")}
         for side in ("left", "right"):
             out.update(part_class("mixer", spec[side].kind).declare(spec[side]))
         return out
@@ -93,8 +101,10 @@ class MixerPair:
         self.right = part_class("mixer", spec["right"].kind)(spec["right"], tensors, device, engine_dtype)
         if self.left.in_dtype != self.right.in_dtype:
             raise ValueError("two mixers side by side read their input in one dtype")
-        self.left_out = place_vector(tensors[n["left_out"]], device)
-        self.right_out = place_vector(tensors[n["right_out"]], device)
+        self.normed = bool(spec.get("normed", True))
+        if self.normed:
+            self.left_out = place_vector(tensors[n["left_out"]], device)
+            self.right_out = place_vector(tensors[n["right_out"]], device)
         self.graph_safe = bool(getattr(self.left, "graph_safe", False) and getattr(self.right, "graph_safe", False))
 
     @property
@@ -113,10 +123,16 @@ class MixerPair:
                 arrays += tuple(FixedArray(prefix + a.name, a.shape, a.dtype, a.init) for a in fixed.all_arrays())
         fixed = FixedSpec(arrays=arrays) if arrays else None
         if paged:
-            return PagedSpec(paged[0].arrays, paged[0].window, fixed, paged[0].chunk)
+            return replace(paged[0], fixed=fixed)
         return fixed
 
     def forward(self, ctx: StepContext, site: int, owns_cache: bool, h: torch.Tensor) -> torch.Tensor:
+        if not self.normed:
+            stream = ctx.stream
+            a = self.left.forward(_Scoped(ctx, "left.", "left:", stream), site, owns_cache, h)
+            b = self.right.forward(_Scoped(ctx, "right.", stream=stream), site, owns_cache, h)
+            deltas = tuple(d for d in (a, b) if stream is None or d is not stream)
+            return stream if not deltas else deltas[0] if len(deltas) == 1 else deltas
         a = self.left.forward(_Scoped(ctx, "left.", "left:"), site, owns_cache, h)
         b = self.right.forward(_Scoped(ctx, "right."), site, owns_cache, h)
         out = ctx.workspace.get("pair_out", (h.shape[0], self.width), torch.float32)

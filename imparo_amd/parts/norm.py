@@ -26,7 +26,7 @@ import torch
 from ..config.plan import PartSpec
 from ..kernels import ops
 from ..weights.loader import TensorDecl
-from .base import Declared, Residual, StepContext
+from .base import Declared, Residual, StepContext, one_delta
 from .linear import place_vector
 from .registry import register_part
 
@@ -74,6 +74,7 @@ class RmsNorm:
         """Adds the pending delta into the stream (if any) and returns the
         normed rows in `out_dtype`."""
         out = ctx.workspace.get(name, tuple(res.x.shape), out_dtype)
+        one_delta(res)
         pending, res.pending = res.pending, None
         post, res.post = res.post, None
         if post is not None and pending is not None:
@@ -96,6 +97,7 @@ class RmsNorm:
         out = ctx.workspace.get(name, tuple(res.x.shape), out_dtype)
         if res.post is not None:
             raise ValueError("the norm with the token shift does not take a sublayer's result through a norm of its own")
+        one_delta(res)
         pending, res.pending = res.pending, None
         ops.group_rms_norm(res.x, self.weight, self.groups, self.eps, out, delta=pending,
                            write_back=pending is not None, shift_mix=mix, shift_state=state, slot=ctx.slot)
@@ -119,6 +121,7 @@ class RmsNorm:
         """Norm of selected rows only (the rows whose logits are wanted); the
         stream itself is left as it is."""
         out = ctx.workspace.get(name, (rows.shape[0], self.width), out_dtype)
+        one_delta(res)
         if res.post is not None and res.pending is not None:
             if self.groups > 1:
                 raise ValueError("a norm in groups cannot take a sublayer's result through a norm of its own")
@@ -128,6 +131,52 @@ class RmsNorm:
         else:
             ops.rms_norm(res.x, self.weight, self.eps, out, delta=res.pending, rows=rows)
         return out
+
+
+class DynamicTanh:
+    """A norm without a statistic: y = tanh(alpha x) * w + b with one number alpha for the whole row, w and b over the
+    row's width. What is pending on the stream, one delta or two, is added in the same launch. Parameters: width,
+    tensor (the weight's name; the others are `<tensor>.alpha`, without dimensions, and `<tensor>.b`)."""
+    role = "norm"
+    graph_safe = True     # launches kernels only: a step made of such parts can be captured
+
+    @staticmethod
+    def _tensors(spec: PartSpec):
+        base = spec.get("tensor") or f"{spec.prefix}.weight"
+        return base, f"{base}.alpha", f"{base}.b"
+
+    @classmethod
+    def declare(cls, spec: PartSpec) -> Declared:
+        w, alpha, b = cls._tensors(spec)
+        return {w: (TensorDecl((spec["width"],), "vector"), "norm"), alpha: (TensorDecl((), "vector"), "norm"),
+                b: (TensorDecl((spec["width"],), "vector"), "bias")}
+
+    def __init__(self, spec: PartSpec, tensors: Dict[str, torch.Tensor], device: torch.device,
+                 engine_dtype: torch.dtype):
+        w, alpha, b = self._tensors(spec)
+        self.width = spec["width"]
+        self.weight, self.bias = place_vector(tensors[w], device), place_vector(tensors[b], device)
+        self.alpha = float(tensors[alpha].to(torch.float32).reshape(()))
+
+    @staticmethod
+    def _deltas(res: Residual):
+        if res.post is not None:
+            raise ValueError("this norm does not take a sublayer's result through a norm of its own")
+        if res.pending is None:
+            return ()
+        return res.pending if isinstance(res.pending, tuple) else (res.pending,)
+
+    def forward(self, ctx: StepContext, res: Residual, out_dtype: torch.dtype, name: str = "normed") -> torch.Tensor:
+        """Adds what is pending into the stream (if anything) and returns the rows behind the norm in `out_dtype`."""
+        out = ctx.workspace.get(name, tuple(res.x.shape), out_dtype)
+        deltas, res.pending = self._deltas(res), None
+        return ops.dynamic_tanh(res.x, self.alpha, self.weight, self.bias, out, deltas, write_back=bool(deltas))
+
+    def forward_rows(self, ctx: StepContext, res: Residual, rows: torch.Tensor, out_dtype: torch.dtype,
+                     name: str = "normed_rows") -> torch.Tensor:
+        """The chosen rows behind the norm; the stream itself is left as it is."""
+        out = ctx.workspace.get(name, (rows.shape[0], self.width), out_dtype)
+        return ops.dynamic_tanh(res.x, self.alpha, self.weight, self.bias, out, self._deltas(res), rows=rows)
 
 
 class NoNorm:
@@ -154,6 +203,7 @@ class NoNorm:
             ops.add_rows(res.x, part)
 
     def forward(self, ctx: StepContext, res: Residual, out_dtype: torch.dtype, name: str = "normed") -> torch.Tensor:
+        one_delta(res)
         pending, res.pending = res.pending, None
         post, res.post = res.post, None
         if pending is not None and post is None:
@@ -171,6 +221,7 @@ class NoNorm:
                      name: str = "normed_rows") -> torch.Tensor:
         """The chosen rows as they would be after the pending add; the stream itself is left as it is."""
         out = ctx.workspace.get(name, (rows.shape[0], self.width), out_dtype)
+        one_delta(res)
         if res.pending is None:
             return ops.cast_rows(res.x, out, rows)
         if res.post is None:
@@ -180,4 +231,5 @@ class NoNorm:
 
 
 register_part("norm", "rms_norm", RmsNorm)
+register_part("norm", "dynamic_tanh", DynamicTanh)
 register_part("norm", "none", NoNorm)

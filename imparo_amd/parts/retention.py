@@ -12,7 +12,13 @@ by side are multiplied by silu(Wg h) and go through the output projection. A
 request's state is S, float32. Angles, the state and every sum of the
 recurrence are float32 whatever the engine's dtype.
 
-Parameters: width, heads, dim, vdim, decay (one number a head), position, eps, names.
+Variations by parameter: `silu_in` (q, k and v go through SiLU; lightning
+attention), `key_scale` (instead of dim^(-1/2)), `norm` (the name of a weight:
+the heads side by side are normed as one row, with that weight, instead of each
+head by itself), `gate` ("silu" or "sigmoid"), `out_scale` (a factor on the
+result, carried in float32 by the rows that the output projection reads).
+
+Parameters: width, heads, dim, vdim, decay (one number a head), position, eps, names, and the above.
 """
 from __future__ import annotations
 
@@ -51,6 +57,7 @@ class Retention:
             n["v"]: (TensorDecl((H * dv, E)), "matrix"),
             n["g"]: (TensorDecl((H * dv, E)), "matrix"),
             n["o"]: (TensorDecl((E, H * dv)), "matrix"),
+            **({f"{spec.prefix}.{spec['norm']}": (TensorDecl((H * dv,), "vector"), "norm")} if spec.get("norm") else {}),
         }
 
     def __init__(self, spec: PartSpec, tensors: Dict[str, torch.Tensor], device: torch.device,
@@ -70,6 +77,17 @@ class Retention:
         # one projection for q | k | v | g: the same dot products, one launch
         self.proj = Linear(place_projection(torch.cat(ws, dim=0), engine_dtype, device))
         self.out = Linear(place_projection(tensors[n["o"]], engine_dtype, device))
+        self.silu_in = bool(spec.get("silu_in"))
+        self.key_scale = float(spec.get("key_scale", float(self.dim) ** -0.5))
+        self.gate = spec.get("gate", "silu")
+        out_scale = float(spec.get("out_scale", 1.0))
+        self.norm, self.norm_groups = None, self.heads
+        if spec.get("norm"):
+            self.norm, self.norm_groups = tensors[f"{spec.prefix}.{spec['norm']}"].to(torch.float32), 1
+        if out_scale != 1.0:        # on the norm's weight, float32
+            self.norm = (torch.ones(self.heads * self.vdim) if self.norm is None else self.norm) * out_scale
+        if self.norm is not None:
+            self.norm = place_vector(self.norm, device)
         pos = spec.get("position") or PartSpec("none")
         self.position = part_class("position", pos.kind)(pos, device)
         if self.position.rotary_dim > self.dim:
@@ -87,12 +105,19 @@ class Retention:
             raise ValueError("a recurrence's state cannot be read from another layer")
         T, H, d, dv = h.shape[0], self.heads, self.dim, self.vdim
         rows = self.proj(ctx, h, torch.float32, "retention_rows", alias="mixer_in")      # q | k | v | g
-        # q and k heads rotated where they lie; the keys carry dim^(-1/2)
-        ops.head_prepare(rows, 0, 2 * H, d, inv_freq=self.position.inv_freq,
-                         interleaved=bool(getattr(self.position, "interleaved", False)), positions=ctx.positions,
-                         n_first=H, scale_first=1.0, scale_rest=float(d) ** -0.5)
+        inv_freq = self.position.inv_freq
+        prepare = inv_freq is not None or self.key_scale != 1.0
         o = ctx.workspace.get("retention_o", (T, H * dv), torch.float32)
         chunk_tokens, max_chunks = ops.decay_scan_chunks(ctx.max_seg_len, dim=d, blocks=ctx.n_rows * H * -(-dv // 8))
+        # SiLU rides in the walk where q, k and v need nothing else and go by token by token
+        silu_walk = self.silu_in and not prepare and not chunk_tokens
+        if self.silu_in and not silu_walk:
+            ops.silu_columns(rows, 0, 2 * H * d + H * dv)
+        if prepare:
+            # q and k heads rotated where they lie; the keys carry their factor
+            ops.head_prepare(rows, 0, 2 * H, d, inv_freq=inv_freq,
+                             interleaved=bool(getattr(self.position, "interleaved", False)), positions=ctx.positions,
+                             n_first=H, scale_first=1.0, scale_rest=self.key_scale)
         chunk_state = chunk_decay = None
         if chunk_tokens:
             n_state, n_decay = ops.decay_scan_scratch(ctx.n_rows, max_chunks, H, d, dv, chunk_tokens)
@@ -100,9 +125,10 @@ class Retention:
             chunk_decay = ctx.workspace.get("scan_chunk_decay", (n_decay,), torch.float32)
         ops.decay_scan(rows, 0, 1, rows, H * d, 1, rows, 2 * H * d, ctx.fixed_arrays(site)["state"], ctx.seg_start,
                        ctx.seg_len, ctx.slot, o, H, d, dv, decay_const=self.decay, chunk_tokens=chunk_tokens,
-                       max_chunks=max_chunks, chunk_state=chunk_state, chunk_decay=chunk_decay)
+                       max_chunks=max_chunks, chunk_state=chunk_state, chunk_decay=chunk_decay, silu_in=silu_walk)
         gated = ctx.workspace.get("retention_gated", (T, H * dv), self.out.in_dtype, alias="mixer_mid")
-        ops.gated_group_norm(o, rows, 2 * H * d + H * dv, None, H, self.eps, gated, gate_first=False)
+        ops.gated_group_norm(o, rows, 2 * H * d + H * dv, self.norm, self.norm_groups, self.eps, gated, gate_first=False,
+                             gate_act=self.gate)
         return self.out(ctx, gated, torch.float32, "mixer_out", sliced_ok=True, into=ctx.stream)
 
 

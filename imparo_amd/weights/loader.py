@@ -25,6 +25,11 @@ from .safetensors_io import SafetensorsError, SafetensorsFile
 WEIGHTS_FILE = "model.safetensors"
 
 
+class FreeDim(int):
+    """A dimension that the file decides (an inner rank that no configuration key names): any positive
+    size is accepted where a declared shape holds one. Its own value is what random-weights mode draws."""
+
+
 @dataclass(frozen=True)
 class TensorDecl:
     shape: Tuple[int, ...]
@@ -135,7 +140,9 @@ def load_weights(model_dir: str, declared: Dict[str, TensorDecl],
     for name in want & have:
         decl = declared[name]
         f = where[name]
-        if tuple(f.shape(name)) != tuple(decl.shape):
+        got = tuple(f.shape(name))
+        if len(got) != len(decl.shape) or any(g != d and not (isinstance(d, FreeDim) and g > 0)
+                                              for g, d in zip(got, decl.shape)):
             wrong_shape.append((name, tuple(decl.shape), tuple(f.shape(name))))
         dt = f.dtype(name)
         ok = dt in _INTS if decl.role == "table" else dt in _FLOATS
