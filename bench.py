@@ -464,6 +464,24 @@ def mepapel_shape(width, heads, expert_ff, dense_ff, experts=8, top=4, layers=16
                 layers=[dict(run[i % 4]) for i in range(layers)])
 
 
+def vebusun_shape(width, heads, ff, layers=16, window=4096, keep_first=64):
+    """A Vebusun model of the width, heads and depth of the Mepapel shape above and its dense feed-forward's width in
+    every layer, in a run of four layers: the channel-decay delta rule (heads of 128 by 128, two heads a query/key
+    head, inner ranks of 128), attention (heads of 64, rotated whole, capped scores, sinks, a window as long as the
+    benchmark's contexts beside the first tokens) beside lightning attention (heads of 128 by 128), the delta rule
+    twice."""
+    wide = width // 128
+    delta = dict(type="channel_delta", mixer=dict(heads=wide, kv_heads=wide // 2, dim=128, vdim=128, conv=4))
+    pair = dict(type="parallel", mixer=dict(
+        left=dict(heads=heads, kv_heads=8, dim=64, vdim=64, scale=0.125, softcap=30.0,
+                  mask=dict(size=window, keep_first=keep_first), rot=dict(dims=64, base=1000000.0)),
+        right=dict(heads=wide, dim=128, vdim=128, decay=[1.0 - 2.0 ** (-5 - 5 * i / max(wide - 1, 1)) for i in range(wide)]),
+        left_scale=0.8, right_scale=0.6))
+    run = [delta, pair, delta, delta]
+    return dict(architecture="Vebusun", vocab=65536, width=width, norm=dict(eps=1e-5), residual_mult=0.5,
+                embedding=dict(scale=1.0), layers=[dict(run[i % 4], mlp=dict(kind="dense", ff=ff)) for i in range(layers)])
+
+
 def compare_workload(workload, sizes, dtype, steps, warmup, beside="lfm2"):
     """Prefill and decode throughput of one design at some sizes, beside the closest model the engine has
     (`beside`: LFM2 unless said) at equal layer sizes, through the same loops. `sizes`: (name, that model's
@@ -545,6 +563,18 @@ def mepapel_workload(dtype, steps, warmup, only=None, alone=False):
     return compare_workload("mepapel", sizes, dtype, steps, warmup, beside="kosalorn")
 
 
+def vebusun_workload(dtype, steps, warmup, only=None, alone=False):
+    """The Vebusun design at two sizes beside Mepapel, the engine's closest model (attention beside linear attention in
+    some layers, the gated delta rule in others), at equal width, heads and depth. `only`: one size; `alone`: without
+    Mepapel."""
+    sizes = [
+        ("1.2B", mepapel_shape(2048, 32, 1408, 5632), vebusun_shape(2048, 32, 5632)),
+        ("350M", mepapel_shape(1024, 16, 768, 3072), vebusun_shape(1024, 16, 3072)),
+    ]
+    sizes = [(n, None if alone else a, b) for n, a, b in sizes if only in (None, n)]
+    return compare_workload("vebusun", sizes, dtype, steps, warmup, beside="mepapel")
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -556,15 +586,16 @@ def main() -> int:
     ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
     ap.add_argument("--no-points", action="store_true", help="skip decode at batch 1 and 64 and the prefill")
     ap.add_argument("--prefill-only", action="store_true", help="run only the 2,048-token prefill (for profiling)")
-    ap.add_argument("--workload", default="decode", choices=["decode", "serving", "long", "tumadra", "pupalorn", "kosalorn", "mepapel"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "serving", "long", "tumadra", "pupalorn", "kosalorn", "mepapel",
+                                                           "vebusun"],
                     help="decode: the headline line (default). serving: continuous batching of 32 requests in 4 "
                          "waves (LFM2-700M shape). long: 64 requests of 32,768-token prompts, then 128 tokens "
                          "each (LFM2-350M shape). tumadra: prefill and decode of the Tumadra design at two sizes "
                          "beside LFM2 at equal size; pupalorn: the same for the Pupalorn design; kosalorn: the "
-                         "Kosalorn design beside Pupalorn; mepapel: the Mepapel design beside Kosalorn. All but the first print "
-                         "a line of their own")
-    ap.add_argument("--size", default=None, choices=["1.2B", "350M"], help="--workload pupalorn, kosalorn or mepapel: one size only")
-    ap.add_argument("--alone", action="store_true", help="--workload pupalorn, kosalorn or mepapel: without the other model's runs beside it")
+                         "Kosalorn design beside Pupalorn; mepapel: the Mepapel design beside Kosalorn; vebusun: the Vebusun "
+                         "design beside Mepapel. All but the first print a line of their own")
+    ap.add_argument("--size", default=None, choices=["1.2B", "350M"], help="--workload pupalorn, kosalorn, mepapel or vebusun: one size only")
+    ap.add_argument("--alone", action="store_true", help="--workload pupalorn, kosalorn, mepapel or vebusun: without the other model's runs beside it")
     ap.add_argument("--requests", type=int, default=64, help="--workload long: concurrent requests")
     ap.add_argument("--prompt-len", type=int, default=32768, help="--workload long: tokens per prompt")
     ap.add_argument("--portion", type=int, default=2048, help="--workload long: tokens of a prompt per step")
@@ -586,6 +617,9 @@ def main() -> int:
         return 0
     if args.workload == "mepapel":
         print(json.dumps(mepapel_workload(args.dtype, args.steps, args.warmup, args.size, args.alone)), flush=True)
+        return 0
+    if args.workload == "vebusun":
+        print(json.dumps(vebusun_workload(args.dtype, args.steps, args.warmup, args.size, args.alone)), flush=True)
         return 0
     if args.workload == "kosalorn":
         print(json.dumps(kosalorn_workload(args.dtype, args.steps, args.warmup, args.size, args.alone)), flush=True)

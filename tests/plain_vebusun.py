@@ -187,15 +187,21 @@ def run_order(cfg: dict) -> List[int]:
     return list(range(loop["start"])) + inside * loop["times"] + list(range(loop["stop"], n))
 
 
-def forward(cfg: dict, w, tokens: List[int], dtype=torch.float64, layers_out: Optional[list] = None, order=None):
-    """Logits [tokens, vocab] of one sequence from position 0."""
+def forward(cfg: dict, w, tokens: List[int], dtype=torch.float64, layers_out: Optional[list] = None, order=None,
+            inputs_as: Optional[torch.dtype] = None):
+    """Logits [tokens, vocab] of one sequence from position 0. `inputs_as`: what every sublayer and the head read is
+    rounded to that dtype first (how much such rounding alone moves the logits)."""
+    def norm(x, name):
+        y = dynamic_tanh(x, w, name)
+        return y if inputs_as is None else y.to(inputs_as).to(y.dtype)
+
     eps, m = cfg["norm"]["eps"], cfg.get("residual_mult", 1.0)
     positions = torch.arange(len(tokens))
     x = w["embed"][torch.tensor(tokens)].to(dtype) * (cfg.get("embedding") or {}).get("scale", 1.0)
     for i in (run_order(cfg) if order is None else order):
         layer = cfg["layers"][i]
         L, kind, mx = f"l{i}", layer["type"], layer["mixer"]
-        h = dynamic_tanh(x, w, f"{L}.norm1")
+        h = norm(x, f"{L}.norm1")
         if kind == "parallel":
             y = side_by_side(h, positions, w, L, mx, eps)
         elif kind == "channel_delta":
@@ -204,10 +210,10 @@ def forward(cfg: dict, w, tokens: List[int], dtype=torch.float64, layers_out: Op
             raise ValueError(kind)
         x = x + m * y
         if layer.get("mlp") is not None:
-            x = x + m * silu_unit(dynamic_tanh(x, w, f"{L}.norm2"), w, f"{L}.mlp")
+            x = x + m * silu_unit(norm(x, f"{L}.norm2"), w, f"{L}.mlp")
         if layers_out is not None:
             layers_out.append(x.clone())
-    return dynamic_tanh(x, w, "final.norm") @ w["head"].T
+    return norm(x, "final.norm") @ w["head"].T
 
 
 class PlainVebusun:
@@ -217,8 +223,9 @@ class PlainVebusun:
         self.dtype = dtype
         self.w = read_tensors(os.path.join(model_dir, "model.safetensors"), dtype)
 
-    def logits(self, tokens: List[int], order=None, layers_out: Optional[list] = None) -> torch.Tensor:
-        return forward(self.cfg, self.w, list(tokens), self.dtype, layers_out, order).to(torch.float32)
+    def logits(self, tokens: List[int], order=None, layers_out: Optional[list] = None,
+               inputs_as: Optional[torch.dtype] = None) -> torch.Tensor:
+        return forward(self.cfg, self.w, list(tokens), self.dtype, layers_out, order, inputs_as).to(torch.float32)
 
     def greedy(self, prompt: List[int], n: int) -> List[int]:
         tokens, out = list(prompt), []
