@@ -247,11 +247,9 @@ __global__ void k_decay_carry(float* __restrict__ chunk_state, const float* __re
 // A first launch makes, for every chunk of every segment and head side by side, T = (I + L)^-1 diag(b) (a lower
 // triangle, by forward substitution, a column a thread), M and the logarithms of g (sums of -rate * step, so
 // that every ratio is the exponential of a difference and at most one). A second launch walks a segment's
-// chunks in order with the state in LDS, a block a (segment, head, run of DVB value columns): four small
-// products a chunk on the vector units, every sum in an order the sizes alone decide. Tokens past a segment's
+// chunks in order: five small products a chunk on the matrix cores, every sum in an order the sizes alone decide. Tokens past a segment's
 // end count as k = q = 0, b = 0 and a decay of one: they change nothing.
 #define DC 32                 // tokens a chunk
-#define DVB 32                // value columns a block of the walk
 #define DMAXK 128             // state rows a head at most, in this form
 
 // PLAIN: the recurrence without the delta rule's correction (b = 1, no triangle): M, log g and the steps only.
@@ -259,7 +257,8 @@ __global__ void k_decay_carry(float* __restrict__ chunk_state, const float* __re
 //   L_tj = b_t sum_i k_ti k_ji g_ti / g_ji,  M_tj = sum_i q_ti k_ji g_ti / g_ji,
 // every ratio the exponential of a difference of logarithms, at most one, so that no decay, however strong, leaves
 // float32's range. The first launch then leaves what the walk multiplies, g_t k_t, g_t q_t, (g_last / g_t) k_t and
-// g_last, beside T and M: T and M [DC, DC], the three [DC, dim4], g_last [dim4], one after the other.
+// g_last, beside T and M: T and M [DC, DC], the first two [DC, DP], the third transposed [DP, DC], g_last [DP], one after
+// the other, DP the state's rows filled up to 64 or 128 with zeros.
 template <bool PLAIN>
 __global__ __launch_bounds__(256) void k_delta_chunk_prepare(const DecayScanArgs A) {
     __shared__ float sk[DC][DMAXK + 1], sq[DC][DMAXK + 1], sL[PLAIN ? 1 : DC][DC + 1], lg[DC], sb[DC];
@@ -339,194 +338,20 @@ __global__ __launch_bounds__(256) void k_delta_chunk_prepare(const DecayScanArgs
     }
 }
 
-// What a block of the walk asks of memory for one chunk, in registers: asked for while the chunk before is worked on.
-#define DPIECES (DC * DMAXK / 256)        // elements of a chunk's K (and Q) a thread brings at most
-struct DeltaFetch {
-    float k[DPIECES], q[DPIECES], t[DC * DC / 256], m[DC * DC / 256], v[DC / 8], dt[DC / 8], l, last;
-};
-
-template <int VB, bool PLAIN>
-__global__ __launch_bounds__(256) void k_delta_chunk_scan(const DecayScanArgs A) {
-    constexpr int KLD = DMAXK + 4;                       // floats between two tokens' rows: whole 16-byte pieces
-    constexpr int NG = 256 / VB;                         // threads a value column: each takes every NG-th token
-    constexpr int TPT = DC / NG;                         // tokens of a chunk a thread takes
-    constexpr int KPT = DMAXK / NG;                      // state rows of its column a thread takes at most
-    __shared__ __attribute__((aligned(16))) float sk[DC][KLD], sq[DC][KLD];
-    __shared__ float sS[DMAXK][VB], sU[DC][VB], sT[PLAIN ? 1 : DC][DC], sM[DC][DC], sg[DC], sw[DC];
-    float (*sR)[VB] = reinterpret_cast<float (*)[VB]>(&sq[0][0]);        // R lies where Q lay, once Q has been used
-    const int r = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VB;
-    const int tid = threadIdx.x, v = tid % VB, g = tid / VB;
-    const int heads = A.heads, dim = A.dim, vdim = A.vdim;
-    const int dim4 = (dim + 3) & ~3;
-    const bool live = v0 + v < vdim;
-    const int n_all = A.seg_len[r], n_chunks = (n_all + DC - 1) / DC;
-    const int qh = h / A.q_div, kh = h / A.k_div;
-    float* S_at = A.state + (((size_t)A.slot[r] * heads + h) * dim) * vdim;
-    for (int i = tid; i < dim4 * VB; i += 256) {
-        const int k = i / VB, c = i - k * VB;
-        sS[k][c] = (k < dim && (v0 + c) < vdim) ? S_at[(size_t)k * vdim + v0 + c] : 0.f;
-    }
-    // which (token, state row) of a chunk's K and Q this thread brings: the same for every chunk
-    int piece_t[DPIECES];
-#pragma unroll
-    for (int it = 0; it < DPIECES; ++it) piece_t[it] = min((tid + 256 * it) / dim4, DC - 1);
-    DeltaFetch f;
-    // every address is clamped into the segment (no load under a branch); what lies beyond is zeroed when it is used
-    auto fetch = [&](int chunk) {
-        const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
-        const size_t at = ((size_t)(r * A.max_chunks + chunk) * heads + h);
-        const float* T_in = A.chunk_state + at * (2 * DC * DC);
-#pragma unroll
-        for (int it = 0; it < DPIECES; ++it) {
-            const int t = piece_t[it], k = min(max(tid + 256 * it - t * dim4, 0), dim - 1);
-            const size_t row = (size_t)(first + min(t, n - 1));
-            f.k[it] = A.k[row * A.k_ld + A.k_off + kh * dim + k];
-            f.q[it] = A.q[row * A.q_ld + A.q_off + qh * dim + k];
-        }
-#pragma unroll
-        for (int it = 0; it < DC * DC / 256; ++it) {
-            if constexpr (!PLAIN) f.t[it] = T_in[tid + 256 * it];
-            f.m[it] = T_in[DC * DC + tid + 256 * it];
-        }
-        f.l = A.chunk_decay[at * (2 * DC) + (tid & (DC - 1))];
-        f.last = A.chunk_decay[at * (2 * DC) + DC - 1];
-#pragma unroll
-        for (int i = 0; i < TPT; ++i) {
-            const int t = min(g + NG * i, n - 1);
-            f.v[i] = A.v[(size_t)(first + t) * A.v_ld + A.v_off + h * vdim + min(v0 + v, vdim - 1)];
-            f.dt[i] = A.chunk_decay[at * (2 * DC) + DC + t];
-        }
-    };
-    fetch(0);
-    const int kpt = (((dim4 + NG - 1) / NG) + 3) & ~3;   // this thread's state rows: kpt from g * kpt on
-    const float skip = (PLAIN && A.skip) ? A.skip[h] : 0.f;
-    for (int chunk = 0; chunk < n_chunks; ++chunk) {
-        const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
-        __syncthreads();                                 // the chunk before has been used, the state is whole
-#pragma unroll
-        for (int it = 0; it < DPIECES; ++it) {
-            const int i = tid + 256 * it, t = piece_t[it], k = i - t * dim4;
-            if (i < DC * dim4) {
-                const bool on = t < n && k < dim;
-                sk[t][k] = on ? f.k[it] : 0.f;
-                sq[t][k] = on ? f.q[it] : 0.f;
-            }
-        }
-#pragma unroll
-        for (int it = 0; it < DC * DC / 256; ++it) {
-            const int i = tid + 256 * it;
-            if constexpr (!PLAIN) sT[i / DC][i % DC] = f.t[it];
-            sM[i / DC][i % DC] = f.m[it];
-        }
-        if (tid < DC) {
-            sg[tid] = expf(f.l);
-            sw[tid] = expf(f.last - f.l);
-        }
-        float vt[TPT], dts[TPT];
-#pragma unroll
-        for (int i = 0; i < TPT; ++i) {
-            vt[i] = (g + NG * i < n && live) ? f.v[i] : 0.f;
-            dts[i] = f.dt[i];
-        }
-        __syncthreads();
-        fetch(min(chunk + 1, n_chunks - 1));             // on its way while this chunk is worked on (no load under a branch)
-        // what the state says of the chunk's keys and queries
-        float p[TPT], s[TPT];
-#pragma unroll
-        for (int i = 0; i < TPT; ++i) p[i] = s[i] = 0.f;
-#pragma unroll 4
-        for (int k = 0; k < dim4; k += 4) {
-            const float s0 = sS[k][v], s1 = sS[k + 1][v], s2 = sS[k + 2][v], s3 = sS[k + 3][v];
-#pragma unroll
-            for (int i = 0; i < TPT; ++i) {
-                const float4 kk = *reinterpret_cast<const float4*>(&sk[g + NG * i][k]);
-                const float4 qq = *reinterpret_cast<const float4*>(&sq[g + NG * i][k]);
-                if constexpr (!PLAIN) p[i] = fmaf(kk.w, s3, fmaf(kk.z, s2, fmaf(kk.y, s1, fmaf(kk.x, s0, p[i]))));
-                s[i] = fmaf(qq.w, s3, fmaf(qq.z, s2, fmaf(qq.y, s1, fmaf(qq.x, s0, s[i]))));
-            }
-        }
-        __syncthreads();                                 // K and Q have been used: R goes where Q lay, K takes its weights
-#pragma unroll
-        for (int i = 0; i < TPT; ++i) {
-            const int t = g + NG * i;
-            if constexpr (PLAIN)
-                sU[t][v] = A.v_times_step ? vt[i] * dts[i] : vt[i];     // no correction: what is written is the value itself
-            else
-                sR[t][v] = vt[i] - sg[t] * p[i];
-            s[i] *= sg[t];
-        }
-        for (int i = tid; i < DC * dim4; i += 256) sk[i / dim4][i % dim4] *= sw[i / dim4];
-        __syncthreads();
-        // (T and M are zero above their diagonals: the sums run over the whole chunk, so that the reads of
-        // several steps can be under way at once; a product with zero adds nothing)
-        if constexpr (!PLAIN) {
-            float u[TPT];
-#pragma unroll
-            for (int i = 0; i < TPT; ++i) u[i] = 0.f;
-#pragma unroll 8
-            for (int j = 0; j < DC; ++j) {
-                const float rv = sR[j][v];
-#pragma unroll
-                for (int i = 0; i < TPT; ++i) u[i] = fmaf(sT[g + NG * i][j], rv, u[i]);
-            }
-#pragma unroll
-            for (int i = 0; i < TPT; ++i) sU[g + NG * i][v] = u[i];
-            __syncthreads();
-        }
-#pragma unroll 8
-        for (int j = 0; j < DC; ++j) {
-            const float uv = sU[j][v];
-#pragma unroll
-            for (int i = 0; i < TPT; ++i) s[i] = fmaf(sM[g + NG * i][j], uv, s[i]);
-        }
-#pragma unroll
-        for (int i = 0; i < TPT; ++i) {
-            const int t = g + NG * i;
-            if (t < n && live)
-                A.out[(size_t)(first + t) * heads * vdim + (size_t)h * vdim + v0 + v] = PLAIN ? fmaf(skip, vt[i], s[i]) : s[i];
-        }
-        // the state behind the chunk: this thread's rows of its column
-        const float g_last = sg[DC - 1];
-        float acc[KPT];
-#pragma unroll
-        for (int m = 0; m < KPT; ++m) acc[m] = (m < kpt && g * kpt + m < dim4) ? g_last * sS[g * kpt + m][v] : 0.f;
-#pragma unroll 4
-        for (int j = 0; j < DC; ++j) {
-            const float u = sU[j][v];
-#pragma unroll
-            for (int m = 0; m < KPT; m += 4)
-                if (m < kpt && g * kpt + m < dim4) {
-                    const float4 w = *reinterpret_cast<const float4*>(&sk[j][g * kpt + m]);
-                    acc[m] = fmaf(w.x, u, acc[m]);
-                    acc[m + 1] = fmaf(w.y, u, acc[m + 1]);
-                    acc[m + 2] = fmaf(w.z, u, acc[m + 2]);
-                    acc[m + 3] = fmaf(w.w, u, acc[m + 3]);
-                }
-        }
-#pragma unroll
-        for (int m = 0; m < KPT; ++m)
-            if (m < kpt && g * kpt + m < dim4) sS[g * kpt + m][v] = acc[m];
-    }
-    __syncthreads();
-    for (int i = tid; i < dim * VB; i += 256) {
-        const int k = i / VB, c = i - k * VB;
-        if (v0 + c < vdim) S_at[(size_t)k * vdim + v0 + c] = sS[k][c];
-    }
-}
-
-__host__ __device__ static inline size_t channel_chunk_floats(int dim4) { return 2 * DC * DC + (3 * DC + 1) * (size_t)dim4; }
+__host__ __device__ static inline size_t channel_chunk_floats(int dp) { return 2 * DC * DC + (3 * DC + 1) * (size_t)dp; }
+__host__ __device__ static inline int channel_rows(int dim) { return dim <= 64 ? 64 : DMAXK; }
 
 __global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanArgs A) {
     __shared__ float sk[DC][DMAXK + 1], sq[DC][DMAXK + 1], lg[DC][DMAXK + 1], sL[DC][DC + 1], sb[DC];
     const int r = blockIdx.x / A.max_chunks, chunk = blockIdx.x - r * A.max_chunks, h = blockIdx.y;
-    const int tid = threadIdx.x, dim = A.dim, heads = A.heads, dim4 = (dim + 3) & ~3;
+    const int tid = threadIdx.x, dim = A.dim, heads = A.heads, dp = channel_rows(dim);
     const int n_all = A.seg_len[r];
     if (chunk * DC >= n_all) return;                     // (the whole block)
     const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
     const int qh = h / A.q_div, kh = h / A.k_div;
-    const float rate = A.rate[h];
-    for (int i = tid; i < DC * dim4; i += 256) {
-        const int t = i / dim4, k = i - t * dim4;
+    const float rate = A.rate[h] * 1.44269504088896340736f;      // logarithms to base 2
+    for (int i = tid; i < DC * dp; i += 256) {
+        const int t = i / dp, k = i - t * dp;
         const bool on = t < n && k < dim;
         const size_t row = (size_t)(first + min(t, n - 1));
         const int kc = min(k, dim - 1);
@@ -539,7 +364,7 @@ __global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanAr
     if (tid < DC)
         sb[tid] = tid < n ? ds_sigmoid(A.beta[(size_t)(first + tid) * A.beta_ld + A.beta_off + h]) : 0.f;
     __syncthreads();
-    if (tid < dim4) {
+    if (tid < dp) {
         float sum = 0.f;
         for (int t = 0; t < DC; ++t) {
             sum += lg[t][tid];
@@ -547,18 +372,18 @@ __global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanAr
         }
     }
     __syncthreads();
-    float* T_out = A.chunk_state + ((size_t)blockIdx.x * heads + h) * channel_chunk_floats(dim4);
+    float* T_out = A.chunk_state + ((size_t)blockIdx.x * heads + h) * channel_chunk_floats(dp);
     float* M_out = T_out + DC * DC;
     float* kg_out = M_out + DC * DC;
-    float* qg_out = kg_out + DC * dim4;
-    float* ke_out = qg_out + DC * dim4;
+    float* qg_out = kg_out + DC * dp;
+    float* ke_out = qg_out + DC * dp;
     for (int i = tid; i < DC * DC; i += 256) {
         const int t = i / DC, j = i - t * DC;
         float kk = 0.f, qk = 0.f;
         if (j <= t) {
 #pragma unroll 4
             for (int k = 0; k < dim; ++k) {
-                const float w = sk[j][k] * expf(lg[t][k] - lg[j][k]);
+                const float w = sk[j][k] * __builtin_amdgcn_exp2f(lg[t][k] - lg[j][k]);
                 kk = fmaf(sk[t][k], w, kk);
                 qk = fmaf(sq[t][k], w, qk);
             }
@@ -566,14 +391,17 @@ __global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanAr
         sL[t][j] = j < t ? kk * sb[t] : 0.f;
         M_out[i] = qk;
     }
-    for (int i = tid; i < DC * dim4; i += 256) {
-        const int t = i / dim4, k = i - t * dim4;
-        const float g = expf(lg[t][k]);
+    for (int i = tid; i < DC * dp; i += 256) {
+        const int t = i / dp, k = i - t * dp;
+        const float g = __builtin_amdgcn_exp2f(lg[t][k]);
         kg_out[i] = sk[t][k] * g;
         qg_out[i] = sq[t][k] * g;
-        ke_out[i] = sk[t][k] * expf(lg[DC - 1][k] - lg[t][k]);
     }
-    if (tid < dim4) ke_out[DC * dim4 + tid] = expf(lg[DC - 1][tid]);
+    for (int i = tid; i < DC * dp; i += 256) {
+        const int k = i / DC, t = i - k * DC;
+        ke_out[i] = sk[t][k] * __builtin_amdgcn_exp2f(lg[DC - 1][k] - lg[t][k]);
+    }
+    if (tid < dp) ke_out[DC * dp + tid] = __builtin_amdgcn_exp2f(lg[DC - 1][tid]);
     __syncthreads();
     if (tid < DC) {
         // column tid of (I + L)^-1 by forward substitution, then times b of that column
@@ -591,155 +419,232 @@ __global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanAr
     }
 }
 
-// The walk: a segment's chunks in order with the state in LDS, a block a (segment, head, run of VB value columns).
-template <int VB>
-__global__ __launch_bounds__(256) void k_channel_delta_scan(const DecayScanArgs A) {
-    constexpr int KLD = DMAXK + 4;                       // floats between two tokens' rows: whole 16-byte pieces
-    constexpr int NG = 256 / VB;                         // threads a value column: each takes every NG-th token
-    constexpr int TPT = DC / NG;                         // tokens of a chunk a thread takes
-    constexpr int KPT = DMAXK / NG;                      // state rows of its column a thread takes at most
-    constexpr int PIECES = DC * DMAXK / 4 / 256;         // 16-byte pieces of a chunk's rows a thread brings at most
-    __shared__ __attribute__((aligned(16))) float sk[DC][KLD], sq[DC][KLD];
-    __shared__ __attribute__((aligned(16))) float sT[DC][DC], sM[DC][DC];
-    __shared__ float sS[DMAXK][VB], sU[DC][VB], gl[DMAXK];
-    float (*sR)[VB] = reinterpret_cast<float (*)[VB]>(&sq[0][0]);        // R lies where Q lay, once Q has been used
-    const int r = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * VB;
-    const int tid = threadIdx.x, v = tid % VB, g = tid / VB;
+// The walk: a segment's chunks in order, a block a (segment, head, run of 16 value columns), every product on the
+// matrix cores in float32 (16x16x4). The state stays in the registers of the result layout: a wave holds TPW of the
+// state's tiles of 16 rows, wave w tiles w, w + 4, ... In that layout a lane of group g = lane / 16 holds rows 4 g + i
+// of its column, and an inner dimension may be walked in any order: taking rows {4 g + i over the groups} as step i makes
+// register i the second operand of the next product as it is, and the first operand 16 neighbouring bytes of a row of K
+// (or Q, T, M). So nothing is staged and nothing moves between lanes; each wave multiplies its own rows of the state,
+// the four partial sums of K S and Q S meet in LDS (two buffers in turn: one barrier a chunk), every wave makes the
+// whole of U for its own update, and waves 0 and 1 finish the 16 results each. The operands of the next chunk are
+// asked for a chunk ahead.
+// KIND: a plain decay (U is V itself), the delta rule, the delta rule with decays a channel (whose operands the first
+// launch has laid out; the others read K and Q where they lie and scale rows of the results instead). VEC: K's and
+// Q's rows can be read in 16-byte pieces.
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+enum { WALK_DELTA = 0, WALK_PLAIN = 1, WALK_CHANNEL = 2 };
+
+template <int KIND, int TPW>
+struct ChunkIn {
+    f32x4 k[2][KIND == WALK_PLAIN ? 1 : TPW], q[2][TPW];   // token 16 a + lane % 16, rows 16 T + 4 g + i of the state
+    f32x4 e[2][TPW];                                       // token 16 a + 4 g + i, row 16 T + lane % 16
+    f32x4 t00, t10, t11, m0, m1;                           // T's three tiles, M's for this wave's results
+    f32x4 gl[KIND == WALK_CHANNEL ? TPW : 1];              // the decay over the chunk, rows 16 T + 4 g + i
+    f32x4 lg[KIND == WALK_CHANNEL ? 1 : 2], dt[KIND == WALK_PLAIN ? 2 : 1], v[2];     // token 16 a + 4 g + i
+    float last;
+};
+
+template <int KIND, int TPW, bool VEC>
+__global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
+    __shared__ f32x4 part[2][4][4][WAVE];                  // [buffer][wave][P of the two halves, Q of the two][lane]
+    const int r = blockIdx.x, h = blockIdx.y;
+    const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE, c = lane & 15, g = lane >> 4;
     const int heads = A.heads, dim = A.dim, vdim = A.vdim;
-    const int dim4 = (dim + 3) & ~3, pieces = DC * dim4 / 4;
-    const bool live = v0 + v < vdim;
-    const int n_all = A.seg_len[r], n_chunks = (n_all + DC - 1) / DC;
-    const size_t floats = channel_chunk_floats(dim4);
+    const int v = blockIdx.z * 16 + c, vc = min(v, vdim - 1);
+    const bool live = v < vdim;
+    const int n_all = A.seg_len[r], n_chunks = (n_all + DC - 1) / DC, start = A.seg_start[r];
+    const int qh = h / A.q_div, kh = h / A.k_div;
     float* S_at = A.state + (((size_t)A.slot[r] * heads + h) * dim) * vdim;
-    for (int i = tid; i < dim4 * VB; i += 256) {
-        const int k = i / VB, c = i - k * VB;
-        sS[k][c] = (k < dim && (v0 + c) < vdim) ? S_at[(size_t)k * vdim + v0 + c] : 0.f;
-    }
-    float4 fk[PIECES], fq[PIECES], fe[PIECES], ft, fm;
-    float fv[TPT], fl;
-    // every address is clamped (no load under a branch)
-    auto fetch = [&](int chunk) {
-        const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
-        const float* at = A.chunk_state + ((size_t)(r * A.max_chunks + chunk) * heads + h) * floats;
-        ft = *reinterpret_cast<const float4*>(at + 4 * tid);
-        fm = *reinterpret_cast<const float4*>(at + DC * DC + 4 * tid);
-        const float* kg = at + 2 * DC * DC;
+    f32x4 S[TPW];
 #pragma unroll
-        for (int it = 0; it < PIECES; ++it) {
-            const int p = min(tid + 256 * it, pieces - 1);
-            fk[it] = *reinterpret_cast<const float4*>(kg + 4 * p);
-            fq[it] = *reinterpret_cast<const float4*>(kg + DC * dim4 + 4 * p);
-            fe[it] = *reinterpret_cast<const float4*>(kg + 2 * DC * dim4 + 4 * p);
+    for (int j = 0; j < TPW; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int k = 16 * (wave + 4 * j) + 4 * g + i;
+            const float x = S_at[(size_t)min(k, dim - 1) * vdim + vc];
+            S[j][i] = (k < dim && live) ? x : 0.f;
         }
-        fl = kg[3 * DC * dim4 + min(tid, dim4 - 1)];
+    // every address is clamped (no load under a branch); tokens past the end repeat the last one and meet zeros in U
+    auto load = [&](ChunkIn<KIND, TPW>& in, int chunk) __attribute__((always_inline)) {
+        chunk = min(chunk, n_chunks - 1);
+        const int first = start + chunk * DC, n = min(DC, n_all - chunk * DC);
+        const size_t at = (size_t)(r * A.max_chunks + chunk) * heads + h;
+        const float* T = A.chunk_state + at * (KIND == WALK_CHANNEL ? channel_chunk_floats(TPW * 64) : (size_t)(2 * DC * DC));
+        const float* M = T + DC * DC;
+        if constexpr (KIND != WALK_PLAIN) {
+            in.t00 = *reinterpret_cast<const f32x4*>(T + c * DC + 4 * g);
+            in.t10 = *reinterpret_cast<const f32x4*>(T + (16 + c) * DC + 4 * g);
+            in.t11 = *reinterpret_cast<const f32x4*>(T + (16 + c) * DC + 16 + 4 * g);
+        }
+        const float* m_row = M + ((wave & 1) * 16 + c) * DC + 4 * g;
+        in.m0 = *reinterpret_cast<const f32x4*>(m_row);
+        in.m1 = *reinterpret_cast<const f32x4*>(m_row + 16);
 #pragma unroll
-        for (int i = 0; i < TPT; ++i) {
-            const int t = min(g + NG * i, n - 1);
-            fv[i] = A.v[(size_t)(first + t) * A.v_ld + A.v_off + h * vdim + min(v0 + v, vdim - 1)];
+        for (int a = 0; a < 2; ++a) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int t = 16 * a + 4 * g + i;
+                const float x = A.v[(size_t)(first + min(t, n - 1)) * A.v_ld + A.v_off + h * vdim + vc];
+                in.v[a][i] = (t < n && live) ? x : 0.f;
+            }
+            if constexpr (KIND == WALK_CHANNEL) {
+                constexpr int DP = TPW * 64;
+                const float* kg = M + DC * DC;
+#pragma unroll
+                for (int j = 0; j < TPW; ++j) {
+                    const int T16 = 16 * (wave + 4 * j);
+                    in.k[a][j] = *reinterpret_cast<const f32x4*>(kg + (16 * a + c) * DP + T16 + 4 * g);
+                    in.q[a][j] = *reinterpret_cast<const f32x4*>(kg + DC * DP + (16 * a + c) * DP + T16 + 4 * g);
+                    in.e[a][j] = *reinterpret_cast<const f32x4*>(kg + 2 * DC * DP + (T16 + c) * DC + 16 * a + 4 * g);
+                    if (a == 0) in.gl[j] = *reinterpret_cast<const f32x4*>(kg + 3 * DC * DP + T16 + 4 * g);
+                }
+            } else {
+                const float* decays = A.chunk_decay + at * (2 * DC);
+                in.lg[a] = *reinterpret_cast<const f32x4*>(decays + 16 * a + 4 * g);
+                if constexpr (KIND == WALK_PLAIN) in.dt[a] = *reinterpret_cast<const f32x4*>(decays + DC + 16 * a + 4 * g);
+                in.last = decays[DC - 1];
+                const size_t row = (size_t)(first + min(16 * a + c, n - 1));
+                const float* kr = A.k + row * A.k_ld + A.k_off + kh * dim;
+                const float* qr = A.q + row * A.q_ld + A.q_off + qh * dim;
+#pragma unroll
+                for (int j = 0; j < TPW; ++j) {
+                    const int k0 = 16 * (wave + 4 * j) + 4 * g, kc = 16 * (wave + 4 * j) + c;
+                    if constexpr (VEC) {                   // (rows of whole pieces: a piece is inside or past the end)
+                        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+                        const f32x4 qv = *reinterpret_cast<const f32x4*>(qr + min(k0, dim - 4));
+                        in.q[a][j] = k0 < dim ? qv : zero;
+                        if constexpr (KIND != WALK_PLAIN) {
+                            const f32x4 kv = *reinterpret_cast<const f32x4*>(kr + min(k0, dim - 4));
+                            in.k[a][j] = k0 < dim ? kv : zero;
+                        }
+                    } else {
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) {
+                            const float qv = qr[min(k0 + i, dim - 1)];
+                            in.q[a][j][i] = k0 + i < dim ? qv : 0.f;
+                            if constexpr (KIND != WALK_PLAIN) {
+                                const float kv = kr[min(k0 + i, dim - 1)];
+                                in.k[a][j][i] = k0 + i < dim ? kv : 0.f;
+                            }
+                        }
+                    }
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const size_t rt = (size_t)(first + min(16 * a + 4 * g + i, n - 1));
+                        const float kv = A.k[rt * A.k_ld + A.k_off + kh * dim + min(kc, dim - 1)];
+                        in.e[a][j][i] = kc < dim ? kv : 0.f;
+                    }
+                }
+            }
         }
     };
-    fetch(0);
-    const int kpt = (((dim4 + NG - 1) / NG) + 3) & ~3;   // this thread's state rows: kpt from g * kpt on
-    for (int chunk = 0; chunk < n_chunks; ++chunk) {
-        const int first = A.seg_start[r] + chunk * DC, n = min(DC, n_all - chunk * DC);
-        __syncthreads();                                 // the chunk before has been used, the state is whole
-        float4 ke[PIECES];
+    auto product = [](const f32x4& x, const f32x4& y, f32x4 acc) __attribute__((always_inline)) {
 #pragma unroll
-        for (int it = 0; it < PIECES; ++it) {
-            const int p = tid + 256 * it, t = p / (dim4 / 4), k = (p - t * (dim4 / 4)) * 4;
-            if (p < pieces) {
-                *reinterpret_cast<float4*>(&sk[t][k]) = fk[it];
-                *reinterpret_cast<float4*>(&sq[t][k]) = fq[it];
+        for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x[i], y[i], acc, 0, 0, 0);
+        return acc;
+    };
+    const float skip = (KIND == WALK_PLAIN && A.skip) ? A.skip[h] : 0.f;
+    auto step = [&](const ChunkIn<KIND, TPW>& in, int chunk) __attribute__((always_inline)) {
+        const int first = start + chunk * DC, n = min(DC, n_all - chunk * DC), buf = chunk & 1;
+        // what the state says of the chunk's keys and queries: this wave's rows of it
+        f32x4 p[2], q[2];
+#pragma unroll
+        for (int a = 0; a < 2; ++a) p[a] = q[a] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if constexpr (KIND != WALK_PLAIN) {
+#pragma unroll
+            for (int j = 0; j < TPW; ++j)
+#pragma unroll
+                for (int a = 0; a < 2; ++a) p[a] = product(in.k[a][j], S[j], p[a]);
+            part[buf][wave][0][lane] = p[0];
+            part[buf][wave][1][lane] = p[1];
+        }
+#pragma unroll
+        for (int j = 0; j < TPW; ++j)
+#pragma unroll
+            for (int a = 0; a < 2; ++a) q[a] = product(in.q[a][j], S[j], q[a]);
+        part[buf][wave][2][lane] = q[0];
+        part[buf][wave][3][lane] = q[1];
+        __syncthreads();
+        f32x4 g_of[2], u[2];
+        if constexpr (KIND != WALK_CHANNEL)
+#pragma unroll
+            for (int a = 0; a < 2; ++a)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) g_of[a][i] = expf(in.lg[a][i]);
+        if constexpr (KIND == WALK_PLAIN) {
+#pragma unroll
+            for (int a = 0; a < 2; ++a) u[a] = A.v_times_step ? in.v[a] * in.dt[a] : in.v[a];
+        } else {
+            f32x4 res[2];
+#pragma unroll
+            for (int a = 0; a < 2; ++a) {
+                f32x4 sum = part[buf][0][a][lane];
+#pragma unroll
+                for (int w = 1; w < 4; ++w) sum = sum + part[buf][w][a][lane];
+                res[a] = KIND == WALK_CHANNEL ? in.v[a] - sum : in.v[a] - g_of[a] * sum;
             }
-            ke[it] = fe[it];
+            const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+            u[0] = product(in.t00, res[0], zero);
+            u[1] = product(in.t11, res[1], product(in.t10, res[0], zero));
         }
-        *reinterpret_cast<float4*>(&sT[tid / (DC / 4)][tid % (DC / 4) * 4]) = ft;
-        *reinterpret_cast<float4*>(&sM[tid / (DC / 4)][tid % (DC / 4) * 4]) = fm;
-        if (tid < dim4) gl[tid] = fl;
-        float vt[TPT];
+        if (wave < 2) {                                    // (the whole wave) results of tokens 16 wave .. + 15
+            f32x4 o = part[buf][0][2 + wave][lane];
 #pragma unroll
-        for (int i = 0; i < TPT; ++i) vt[i] = (g + NG * i < n && live) ? fv[i] : 0.f;
-        __syncthreads();
-        fetch(min(chunk + 1, n_chunks - 1));             // on its way while this chunk is worked on (no load under a branch)
-        // what the decayed state says of the chunk's keys and queries
-        float p[TPT], s[TPT];
+            for (int w = 1; w < 4; ++w) o = o + part[buf][w][2 + wave][lane];
+            if constexpr (KIND != WALK_CHANNEL) o = o * (wave ? g_of[1] : g_of[0]);
+            o = product(in.m0, u[0], o);
+            if (wave) o = product(in.m1, u[1], o);
+            if (KIND == WALK_PLAIN && skip != 0.f) o = o + skip * (wave ? in.v[1] : in.v[0]);
 #pragma unroll
-        for (int i = 0; i < TPT; ++i) p[i] = s[i] = 0.f;
-#pragma unroll 4
-        for (int k = 0; k < dim4; k += 4) {
-            const float s0 = sS[k][v], s1 = sS[k + 1][v], s2 = sS[k + 2][v], s3 = sS[k + 3][v];
-#pragma unroll
-            for (int i = 0; i < TPT; ++i) {
-                const float4 kk = *reinterpret_cast<const float4*>(&sk[g + NG * i][k]);
-                const float4 qq = *reinterpret_cast<const float4*>(&sq[g + NG * i][k]);
-                p[i] = fmaf(kk.w, s3, fmaf(kk.z, s2, fmaf(kk.y, s1, fmaf(kk.x, s0, p[i]))));
-                s[i] = fmaf(qq.w, s3, fmaf(qq.z, s2, fmaf(qq.y, s1, fmaf(qq.x, s0, s[i]))));
+            for (int i = 0; i < 4; ++i) {
+                const int t = 16 * wave + 4 * g + i;
+                if (t < n && live) A.out[(size_t)(first + t) * heads * vdim + (size_t)h * vdim + v] = o[i];
             }
         }
-        __syncthreads();                                 // K and Q have been used: R goes where Q lay, the weighed keys where K lay
+        // the state behind the chunk
+        if constexpr (KIND != WALK_CHANNEL) {
+            const float g_last = expf(in.last);
 #pragma unroll
-        for (int i = 0; i < TPT; ++i) sR[g + NG * i][v] = vt[i] - p[i];
+            for (int a = 0; a < 2; ++a)
 #pragma unroll
-        for (int it = 0; it < PIECES; ++it) {
-            const int pc = tid + 256 * it, t = pc / (dim4 / 4), k = (pc - t * (dim4 / 4)) * 4;
-            if (pc < pieces) *reinterpret_cast<float4*>(&sk[t][k]) = ke[it];
-        }
-        __syncthreads();
-        // (T and M are zero above their diagonals: the sums run over the whole chunk, so that the reads of
-        // several steps can be under way at once; a product with zero adds nothing)
-        float u[TPT];
+                for (int i = 0; i < 4; ++i) u[a][i] *= expf(in.last - in.lg[a][i]);
 #pragma unroll
-        for (int i = 0; i < TPT; ++i) u[i] = 0.f;
-#pragma unroll 8
-        for (int j = 0; j < DC; ++j) {
-            const float rv = sR[j][v];
+            for (int j = 0; j < TPW; ++j) S[j] = S[j] * g_last;
+        } else {
 #pragma unroll
-            for (int i = 0; i < TPT; ++i) u[i] = fmaf(sT[g + NG * i][j], rv, u[i]);
+            for (int j = 0; j < TPW; ++j) S[j] = S[j] * in.gl[j];
         }
 #pragma unroll
-        for (int i = 0; i < TPT; ++i) sU[g + NG * i][v] = u[i];
-        __syncthreads();
-#pragma unroll 8
-        for (int j = 0; j < DC; ++j) {
-            const float uv = sU[j][v];
+        for (int j = 0; j < TPW; ++j)
 #pragma unroll
-            for (int i = 0; i < TPT; ++i) s[i] = fmaf(sM[g + NG * i][j], uv, s[i]);
-        }
-#pragma unroll
-        for (int i = 0; i < TPT; ++i) {
-            const int t = g + NG * i;
-            if (t < n && live) A.out[(size_t)(first + t) * heads * vdim + (size_t)h * vdim + v0 + v] = s[i];
-        }
-        // the state behind the chunk: this thread's rows of its column
-        float acc[KPT];
-#pragma unroll
-        for (int m = 0; m < KPT; ++m)
-            acc[m] = (m < kpt && g * kpt + m < dim4) ? gl[g * kpt + m] * sS[g * kpt + m][v] : 0.f;
-#pragma unroll 4
-        for (int j = 0; j < DC; ++j) {
-            const float uv = sU[j][v];
-#pragma unroll
-            for (int m = 0; m < KPT; m += 4)
-                if (m < kpt && g * kpt + m < dim4) {
-                    const float4 w = *reinterpret_cast<const float4*>(&sk[j][g * kpt + m]);
-                    acc[m] = fmaf(w.x, uv, acc[m]);
-                    acc[m + 1] = fmaf(w.y, uv, acc[m + 1]);
-                    acc[m + 2] = fmaf(w.z, uv, acc[m + 2]);
-                    acc[m + 3] = fmaf(w.w, uv, acc[m + 3]);
-                }
-        }
-#pragma unroll
-        for (int m = 0; m < KPT; ++m)
-            if (m < kpt && g * kpt + m < dim4) sS[g * kpt + m][v] = acc[m];
+            for (int a = 0; a < 2; ++a) S[j] = product(in.e[a][j], u[a], S[j]);
+    };
+    ChunkIn<KIND, TPW> even, odd;
+    load(even, 0);
+    for (int chunk = 0; chunk < n_chunks; chunk += 2) {
+        load(odd, chunk + 1);
+        step(even, chunk);
+        if (chunk + 1 >= n_chunks) break;
+        load(even, chunk + 2);
+        step(odd, chunk + 1);
     }
-    __syncthreads();
-    for (int i = tid; i < dim * VB; i += 256) {
-        const int k = i / VB, c = i - k * VB;
-        if (v0 + c < vdim) S_at[(size_t)k * vdim + v0 + c] = sS[k][c];
-    }
+#pragma unroll
+    for (int j = 0; j < TPW; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int k = 16 * (wave + 4 * j) + 4 * g + i;
+            if (k < dim && live) S_at[(size_t)k * vdim + v] = S[j][i];
+        }
 }
 
-extern "C" long long imparo_channel_delta_scratch(int dim) { return (long long)channel_chunk_floats((dim + 3) & ~3); }
+template <int KIND, bool VEC>
+static void launch_walk(const DecayScanArgs& args, int n_rows, hipStream_t s) {
+    const dim3 grid(n_rows, args.heads, (args.vdim + 15) / 16);
+    if (args.dim <= 64) k_chunk_walk<KIND, 1, VEC><<<grid, 256, 0, s>>>(args);
+    else k_chunk_walk<KIND, 2, VEC><<<grid, 256, 0, s>>>(args);
+}
+
+extern "C" long long imparo_channel_delta_scratch(int dim) { return (long long)channel_chunk_floats(channel_rows(dim)); }
 
 extern "C" int imparo_channel_delta_scan(const float* q, int q_ld, int q_off, int q_div, const float* k, int k_ld,
                                          int k_off, int k_div, const float* v, int v_ld, int v_off, const float* step,
@@ -775,13 +680,7 @@ extern "C" int imparo_channel_delta_scan(const float* q, int q_ld, int q_off, in
     args.chunk_tokens = chunk_tokens, args.max_chunks = max_chunks, args.chunk_state = scratch;
     if (chunk_tokens) {
         k_channel_delta_prepare<<<dim3(n_rows * max_chunks, heads), 256, 0, s>>>(args);
-        // few blocks (a segment, few heads): narrower runs of columns make more of them
-        const long long rh = (long long)n_rows * heads;
-#define CDS(VB) k_channel_delta_scan<VB><<<dim3(n_rows, heads, (vdim + VB - 1) / VB), 256, 0, s>>>(args)
-        if (rh * ((vdim + 31) / 32) >= 512) CDS(32);
-        else if (rh * ((vdim + 15) / 16) >= 512) CDS(16);
-        else CDS(8);
-#undef CDS
+        launch_walk<WALK_CHANNEL, true>(args, n_rows, s);
         return launch_status();
     }
     int threads = (ks * vdim + WAVE - 1) / WAVE * WAVE;
@@ -822,7 +721,7 @@ extern "C" int imparo_decay_scan(const float* q, int q_ld, int q_off, int q_div,
     if (chunk_tokens < 0 || chunk_tokens % DS_TOKENS) return IMPARO_BAD_ARGUMENT;
     if (chunk_tokens && (max_chunks < 1 || !chunk_state || !chunk_decay)) return IMPARO_BAD_ARGUMENT;
     if (chunk_tokens && beta && (chunk_tokens != DC || dim > DMAXK || decay_const)) return IMPARO_BAD_ARGUMENT;
-    if (chunk_tokens == DC && dim > DMAXK) return IMPARO_BAD_ARGUMENT;
+    if (chunk_tokens == DC && (dim > DMAXK || (((uintptr_t)chunk_state | (uintptr_t)chunk_decay) & 15))) return IMPARO_BAD_ARGUMENT;
     if (n_rows < 0 || heads < 1 || dim < 1 || dim > DS_MAX_DIM || vdim < 1) return IMPARO_BAD_ARGUMENT;
     if (q_div < 1 || k_div < 1 || heads % q_div || heads % k_div) return IMPARO_BAD_ARGUMENT;
     if (q_off < 0 || k_off < 0 || v_off < 0 || q_ld < q_off + heads / q_div * dim || k_ld < k_off + heads / k_div * dim ||
@@ -853,16 +752,12 @@ extern "C" int imparo_decay_scan(const float* q, int q_ld, int q_off, int q_div,
         const dim3 pgrid(n_rows * max_chunks, heads);
         if (beta) k_delta_chunk_prepare<false><<<pgrid, 256, 0, s>>>(args);
         else k_delta_chunk_prepare<true><<<pgrid, 256, 0, s>>>(args);
-        // few blocks (a segment, few heads): narrower runs of columns make more of them
-        // (a column's arithmetic is the same whatever the width of its run: the same bits)
-        const long long rh = (long long)n_rows * heads;
-#define DCS(VB)                                                                                                      \
-    if (beta) k_delta_chunk_scan<VB, false><<<dim3(n_rows, heads, (vdim + VB - 1) / VB), 256, 0, s>>>(args);        \
-    else k_delta_chunk_scan<VB, true><<<dim3(n_rows, heads, (vdim + VB - 1) / VB), 256, 0, s>>>(args)
-        if (rh * ((vdim + DVB - 1) / DVB) >= 512 || vdim <= 8) { DCS(DVB); }
-        else if (rh * ((vdim + 15) / 16) >= 512) { DCS(16); }
-        else { DCS(8); }
-#undef DCS
+        const bool vec = dim % 4 == 0 && q_ld % 4 == 0 && q_off % 4 == 0 && k_ld % 4 == 0 && k_off % 4 == 0 &&
+                         !(((uintptr_t)q | (uintptr_t)k) & 15);
+        if (beta && vec) launch_walk<WALK_DELTA, true>(args, n_rows, s);
+        else if (beta) launch_walk<WALK_DELTA, false>(args, n_rows, s);
+        else if (vec) launch_walk<WALK_PLAIN, true>(args, n_rows, s);
+        else launch_walk<WALK_PLAIN, false>(args, n_rows, s);
         return launch_status();
     }
 #define DS_PASS(KS, MODE, DELTA)                                                                                     \
