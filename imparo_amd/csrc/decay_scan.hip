@@ -377,19 +377,26 @@ __global__ __launch_bounds__(256) void k_channel_delta_prepare(const DecayScanAr
     float* kg_out = M_out + DC * DC;
     float* qg_out = kg_out + DC * dp;
     float* ke_out = qg_out + DC * dp;
-    for (int i = tid; i < DC * DC; i += 256) {
+    for (int i = tid; i < DC * DC; i += 256) {             // above the diagonals
         const int t = i / DC, j = i - t * DC;
+        if (j >= t) sL[t][j] = 0.f;
+        if (j > t) M_out[i] = 0.f;
+    }
+    // the pairs j <= t one after the other, row by row, so that no lane idles on the other half of the square
+    for (int p = tid; p < DC * (DC + 1) / 2; p += 256) {
+        int t = (int)((sqrtf(8.0f * (float)p + 1.0f) - 1.0f) * 0.5f);
+        if (t * (t + 1) / 2 > p) --t;
+        if ((t + 1) * (t + 2) / 2 <= p) ++t;
+        const int j = p - t * (t + 1) / 2;
         float kk = 0.f, qk = 0.f;
-        if (j <= t) {
-#pragma unroll 4
-            for (int k = 0; k < dim; ++k) {
-                const float w = sk[j][k] * __builtin_amdgcn_exp2f(lg[t][k] - lg[j][k]);
-                kk = fmaf(sk[t][k], w, kk);
-                qk = fmaf(sq[t][k], w, qk);
-            }
+#pragma unroll 8
+        for (int k = 0; k < dim; ++k) {
+            const float w = sk[j][k] * __builtin_amdgcn_exp2f(lg[t][k] - lg[j][k]);
+            kk = fmaf(sk[t][k], w, kk);
+            qk = fmaf(sq[t][k], w, qk);
         }
-        sL[t][j] = j < t ? kk * sb[t] : 0.f;
-        M_out[i] = qk;
+        if (j < t) sL[t][j] = kk * sb[t];
+        M_out[t * DC + j] = qk;
     }
     for (int i = tid; i < DC * dp; i += 256) {
         const int t = i / dp, k = i - t * dp;
@@ -464,7 +471,8 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
             const float x = S_at[(size_t)min(k, dim - 1) * vdim + vc];
             S[j][i] = (k < dim && live) ? x : 0.f;
         }
-    // every address is clamped (no load under a branch); tokens past the end repeat the last one and meet zeros in U
+    // every address is clamped and nothing is chosen here (no load may end up under a branch); tokens past the end
+    // repeat the last one and meet zeros in U
     auto load = [&](ChunkIn<KIND, TPW>& in, int chunk) __attribute__((always_inline)) {
         chunk = min(chunk, n_chunks - 1);
         const int first = start + chunk * DC, n = min(DC, n_all - chunk * DC);
@@ -485,7 +493,7 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
             for (int i = 0; i < 4; ++i) {
                 const int t = 16 * a + 4 * g + i;
                 const float x = A.v[(size_t)(first + min(t, n - 1)) * A.v_ld + A.v_off + h * vdim + vc];
-                in.v[a][i] = (t < n && live) ? x : 0.f;
+                in.v[a][i] = x;
             }
             if constexpr (KIND == WALK_CHANNEL) {
                 constexpr int DP = TPW * 64;
@@ -509,30 +517,21 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
 #pragma unroll
                 for (int j = 0; j < TPW; ++j) {
                     const int k0 = 16 * (wave + 4 * j) + 4 * g, kc = 16 * (wave + 4 * j) + c;
-                    if constexpr (VEC) {                   // (rows of whole pieces: a piece is inside or past the end)
-                        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-                        const f32x4 qv = *reinterpret_cast<const f32x4*>(qr + min(k0, dim - 4));
-                        in.q[a][j] = k0 < dim ? qv : zero;
-                        if constexpr (KIND != WALK_PLAIN) {
-                            const f32x4 kv = *reinterpret_cast<const f32x4*>(kr + min(k0, dim - 4));
-                            in.k[a][j] = k0 < dim ? kv : zero;
-                        }
+                    // (past dim: other numbers of the row, which meet state rows that stay zero)
+                    if constexpr (VEC) {                   // rows of whole pieces
+                        in.q[a][j] = *reinterpret_cast<const f32x4*>(qr + min(k0, dim - 4));
+                        if constexpr (KIND != WALK_PLAIN) in.k[a][j] = *reinterpret_cast<const f32x4*>(kr + min(k0, dim - 4));
                     } else {
 #pragma unroll
                         for (int i = 0; i < 4; ++i) {
-                            const float qv = qr[min(k0 + i, dim - 1)];
-                            in.q[a][j][i] = k0 + i < dim ? qv : 0.f;
-                            if constexpr (KIND != WALK_PLAIN) {
-                                const float kv = kr[min(k0 + i, dim - 1)];
-                                in.k[a][j][i] = k0 + i < dim ? kv : 0.f;
-                            }
+                            in.q[a][j][i] = qr[min(k0 + i, dim - 1)];
+                            if constexpr (KIND != WALK_PLAIN) in.k[a][j][i] = kr[min(k0 + i, dim - 1)];
                         }
                     }
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
                         const size_t rt = (size_t)(first + min(16 * a + 4 * g + i, n - 1));
-                        const float kv = A.k[rt * A.k_ld + A.k_off + kh * dim + min(kc, dim - 1)];
-                        in.e[a][j][i] = kc < dim ? kv : 0.f;
+                        in.e[a][j][i] = A.k[rt * A.k_ld + A.k_off + kh * dim + min(kc, dim - 1)];
                     }
                 }
             }
@@ -565,7 +564,11 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
         part[buf][wave][2][lane] = q[0];
         part[buf][wave][3][lane] = q[1];
         __syncthreads();
-        f32x4 g_of[2], u[2];
+        f32x4 g_of[2], u[2], vv[2];
+#pragma unroll
+        for (int a = 0; a < 2; ++a)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) vv[a][i] = (16 * a + 4 * g + i < n && live) ? in.v[a][i] : 0.f;
         if constexpr (KIND != WALK_CHANNEL)
 #pragma unroll
             for (int a = 0; a < 2; ++a)
@@ -573,7 +576,7 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
                 for (int i = 0; i < 4; ++i) g_of[a][i] = expf(in.lg[a][i]);
         if constexpr (KIND == WALK_PLAIN) {
 #pragma unroll
-            for (int a = 0; a < 2; ++a) u[a] = A.v_times_step ? in.v[a] * in.dt[a] : in.v[a];
+            for (int a = 0; a < 2; ++a) u[a] = A.v_times_step ? vv[a] * in.dt[a] : vv[a];
         } else {
             f32x4 res[2];
 #pragma unroll
@@ -581,7 +584,7 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
                 f32x4 sum = part[buf][0][a][lane];
 #pragma unroll
                 for (int w = 1; w < 4; ++w) sum = sum + part[buf][w][a][lane];
-                res[a] = KIND == WALK_CHANNEL ? in.v[a] - sum : in.v[a] - g_of[a] * sum;
+                res[a] = KIND == WALK_CHANNEL ? vv[a] - sum : vv[a] - g_of[a] * sum;
             }
             const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
             u[0] = product(in.t00, res[0], zero);
@@ -594,7 +597,7 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
             if constexpr (KIND != WALK_CHANNEL) o = o * (wave ? g_of[1] : g_of[0]);
             o = product(in.m0, u[0], o);
             if (wave) o = product(in.m1, u[1], o);
-            if (KIND == WALK_PLAIN && skip != 0.f) o = o + skip * (wave ? in.v[1] : in.v[0]);
+            if (KIND == WALK_PLAIN && skip != 0.f) o = o + skip * (wave ? vv[1] : vv[0]);
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int t = 16 * wave + 4 * g + i;
@@ -617,7 +620,13 @@ __global__ __launch_bounds__(256) void k_chunk_walk(const DecayScanArgs A) {
 #pragma unroll
         for (int j = 0; j < TPW; ++j)
 #pragma unroll
-            for (int a = 0; a < 2; ++a) S[j] = product(in.e[a][j], u[a], S[j]);
+            for (int a = 0; a < 2; ++a) {
+                f32x4 e = in.e[a][j];
+                if constexpr (KIND != WALK_CHANNEL)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) e[i] = 16 * (wave + 4 * j) + c < dim ? e[i] : 0.f;
+                S[j] = product(e, u[a], S[j]);
+            }
     };
     ChunkIn<KIND, TPW> even, odd;
     load(even, 0);
