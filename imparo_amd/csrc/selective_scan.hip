@@ -42,6 +42,48 @@ __global__ void k_causal_conv(const float* __restrict__ u, int u_ld, const float
     store_f32<TOut>(out, (size_t)t * channels + c, silu ? silu_f32(acc) : acc);
 }
 
+// The same for filters of a few taps over many tokens: a thread takes CONV_TILE tokens of a channel, its weights once
+// and its inputs once, all asked for before any is used. Tokens whose window starts before their segment take the
+// missing inputs from the history (the same for the whole block).
+#define CONV_TILE 8
+template <typename TOut, int TAPS>
+__global__ void k_causal_conv_tile(const float* __restrict__ u, int u_ld, const float* __restrict__ weight,
+                                   const float* __restrict__ bias, const float* __restrict__ state,
+                                   const int32_t* __restrict__ row_of_token, const int32_t* __restrict__ seg_start,
+                                   const int32_t* __restrict__ slot, TOut* __restrict__ out, int n_tokens, int channels,
+                                   int silu) {
+    const int c = blockIdx.y * blockDim.x + threadIdx.x;
+    const int first = blockIdx.x * CONV_TILE;
+    if (c >= channels) return;
+    constexpr int history = TAPS - 1;
+    float x[CONV_TILE + history], w[TAPS];
+#pragma unroll
+    for (int i = 0; i < CONV_TILE + history; ++i)
+        x[i] = u[(size_t)min(max(first - history + i, 0), n_tokens - 1) * u_ld + c];
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) w[k] = weight[(size_t)c * TAPS + k];
+    const float b = bias ? bias[c] : 0.f;
+#pragma unroll
+    for (int i = 0; i < CONV_TILE; ++i) {
+        const int t = first + i;
+        if (t >= n_tokens) return;
+        const int r = row_of_token[t], t0 = seg_start[r];
+        float acc = b;
+        if (t - history >= t0) {
+#pragma unroll
+            for (int k = 0; k < TAPS; ++k) acc += w[k] * x[i + k];
+        } else {
+            const float* st = state + (size_t)slot[r] * history * channels;
+#pragma unroll
+            for (int k = 0; k < TAPS; ++k) {
+                const int src = t - (history - k);
+                acc += w[k] * (src >= t0 ? x[i + k] : st[(size_t)(history - (t0 - src)) * channels + c]);
+            }
+        }
+        store_f32<TOut>(out, (size_t)t * channels + c, silu ? silu_f32(acc) : acc);
+    }
+}
+
 // One thread per (request, channel) owns that channel's whole history, so the update is race-free in
 // place: it reads every value it needs before it writes. Works for segments shorter than the history.
 __global__ void k_causal_conv_state(const float* __restrict__ u, int u_ld, float* __restrict__ state,
@@ -109,7 +151,20 @@ extern "C" int imparo_causal_conv(const float* u, int u_ld, const float* weight,
         return launch_status();
     }
     dim3 grid(n_tokens, cb);
-    if (out_dtype == IMPARO_F32)
+    const bool tiled = n_tokens >= 64 && taps >= 2 && taps <= 4;
+    if (tiled) {
+        const dim3 tiles((n_tokens + CONV_TILE - 1) / CONV_TILE, cb);
+#define CONV_TILED(T, TAPS)                                                                                          \
+    k_causal_conv_tile<T, TAPS><<<tiles, threads, 0, s>>>(u, u_ld, weight, bias, state, row_of_token, seg_start, slot, \
+                                                          (T*)out, n_tokens, channels, silu)
+#define CONV_TAPS(T)                                                                                                 \
+    if (taps == 2) CONV_TILED(T, 2);                                                                                 \
+    else if (taps == 3) CONV_TILED(T, 3);                                                                            \
+    else CONV_TILED(T, 4)
+        if (out_dtype == IMPARO_F32) { CONV_TAPS(float); } else { CONV_TAPS(bf16_t); }
+#undef CONV_TAPS
+#undef CONV_TILED
+    } else if (out_dtype == IMPARO_F32)
         k_causal_conv<float><<<grid, threads, 0, s>>>(u, u_ld, weight, bias, state, row_of_token, seg_start, slot,
                                                       (float*)out, channels, taps, silu);
     else

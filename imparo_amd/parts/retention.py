@@ -108,7 +108,7 @@ class Retention:
         inv_freq = self.position.inv_freq
         prepare = inv_freq is not None or self.key_scale != 1.0
         o = ctx.workspace.get("retention_o", (T, H * dv), torch.float32)
-        chunk_tokens, max_chunks = ops.decay_scan_chunks(ctx.max_seg_len, dim=d, blocks=ctx.n_rows * H * -(-dv // 8))
+        chunk_tokens, max_chunks = ops.decay_scan_chunks(ctx.max_seg_len, dim=d, blocks=ctx.n_rows * H * -(-dv // 16))
         # SiLU rides in the walk where q, k and v need nothing else and go by token by token
         silu_walk = self.silu_in and not prepare and not chunk_tokens
         if self.silu_in and not silu_walk:

@@ -674,3 +674,34 @@ def test_trace_replay_program(dirs, plains, tmp_path):
     check_logits(read(0), ref[[0, 19]], "float32", "step 0")
     check_logits(read(1), ref_other[[8]], "float32", "step 1")
     check_logits(read(2), ref[[44]], "float32", "step 2")
+
+
+@pytest.mark.parametrize("taps", [2, 3, 4])
+@pytest.mark.parametrize("out_dtype", [torch.float32, torch.bfloat16])
+def test_short_conv_over_many_tokens(taps, out_dtype):
+    """Segments of many sizes in one batch of many tokens, so that runs of tokens that share their loads hold the end of
+    one segment and the start of another, beside histories left by earlier batches."""
+    from imparo_amd.kernels import ops
+    g = torch.Generator().manual_seed(taps)
+    C, ld, off, slots = 70, 90, 3, [4, 1, 0, 6, 2]
+    cuts = [[1, 70, 2], [3, 9, 65], [33, 1, 1], [50, 5, 17], [2, 2, 40]]
+    w = torch.randn(C, taps, generator=g)
+    rows = [torch.randn(sum(cut), ld, generator=g) for cut in cuts]
+    want = [plain.silu(plain.causal_conv(x[:, off:off + C].double(), w.double())) for x in rows]
+    st = dev(torch.randn(7, taps - 1, C, generator=g))
+    for s in slots:
+        st[s].zero_()
+    got, fed = [[] for _ in cuts], [0] * len(cuts)
+    for step in range(3):
+        seg = [cut[step] for cut in cuts]
+        u = dev(torch.cat([x[f:f + n] for x, f, n in zip(rows, fed, seg)]))
+        assert u.shape[0] >= 64
+        row_of = np.concatenate([[i] * n for i, n in enumerate(seg)])
+        out = torch.empty(u.shape[0], C, dtype=out_dtype, device=DEV)
+        ops.causal_conv(u, C, dev(w), None, st, i32(row_of), i32(np.cumsum([0] + seg[:-1])), i32(seg), i32(slots), out, silu=True,
+                        u_off=off)
+        for i, o in enumerate(torch.split(out.float().cpu(), seg)):
+            got[i].append(o)
+            fed[i] += seg[i]
+    for i in range(len(cuts)):
+        near(torch.cat(got[i]), want[i], 3e-6 if out_dtype == torch.float32 else 5e-3, f"request {i}")
